@@ -144,6 +144,7 @@ class RequestCache:
         self.slot = slot
         self.length = 0
         self.blocks: List[List[int]] = [[] for _ in range(n_paged_groups)]  # -1 = given back
+        self.passed = [0] * n_paged_groups   # the first block a window has not looked past yet
         self.closed = False
         self.version = 0        # counts changes of `blocks`, for callers that mirror them
         self._arrays = [(-1, None)] * n_paged_groups      # (version, blocks[g] as int32 array)
@@ -320,7 +321,8 @@ class CacheManager:
 
     def dump(self, rc: RequestCache) -> dict:
         """Everything the request holds, for debugging: its length, slot and block tables, and
-        per cache id what ``export_range`` (the positions still kept) or ``export_state`` gives."""
+        per cache id what ``export_range`` (the positions still in the window; under "kept" the
+        first tokens of a group that keeps them) or ``export_state`` gives."""
         self._check_live(rc)
         out = {"request": rc.request_id, "length": rc.length, "slot": rc.slot,
                "blocks": [list(b) for b in rc.blocks], "caches": {}}
@@ -329,10 +331,13 @@ class CacheManager:
             if kind == "state":
                 out["caches"][cid] = {"kind": "state", "state": self.export_state(rc, cid)}
                 continue
-            first = next((i for i, b in enumerate(rc.blocks[gi]) if b >= 0), 0) * self.page_size
-            first = min(first, rc.length)
+            gone = [i for i, b in enumerate(rc.blocks[gi]) if b < 0]
+            first = min((gone[-1] + 1) * self.page_size if gone else 0, rc.length)
             out["caches"][cid] = {"kind": "paged", "first_position": first,
                                   **self.export_range(rc, cid, first, rc.length - first)}
+            kept = min(self.paged_groups[gi].spec.keep_first, first)
+            if kept:
+                out["caches"][cid]["kept"] = self.export_range(rc, cid, 0, kept)
         return out
 
     # -- requests -------------------------------------------------------------------------
@@ -418,7 +423,8 @@ class CacheManager:
 
     def commit(self, rc: RequestCache, n_new: int) -> None:
         """The step has stored ``n_new`` tokens.  Pages that no later position can see
-        through its window go back to the pool."""
+        through its window go back to the pool, but for those of the first tokens that the
+        group keeps."""
         self._check_live(rc)
         rc.length += n_new
         if self._blocks_for(rc.length) > min((len(b) for b in rc.blocks), default=10 ** 18):
@@ -428,13 +434,14 @@ class CacheManager:
             if not w:
                 continue
             first_needed = rc.length - w + 1      # oldest key a query at position >= length sees
-            b = 0
+            b = max(self._blocks_for(g.spec.keep_first), rc.passed[gi])
             while (b + 1) * self.page_size <= first_needed and b < len(rc.blocks[gi]):
                 if rc.blocks[gi][b] >= 0:
                     g.allocator.give_back(rc.blocks[gi][b], rc.request_id)
                     rc.blocks[gi][b] = -1
                     rc.version += 1
                 b += 1
+            rc.passed[gi] = b
 
     def trim_uncommitted(self, rc: RequestCache) -> None:
         """Give back pages that ``extend`` took for tokens that were never committed."""

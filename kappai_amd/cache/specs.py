@@ -29,10 +29,13 @@ class PagedSpec:
     ``window``          None keeps every token; a number keeps only what the last ``window``
                         positions can still see, and pages that have fallen out of every future
                         window are given back;
+    ``keep_first``      with a window: the first that many tokens of a sequence stay, and so do
+                        the pages they lie in;
     ``pools(page_size)``        the tensors of a page, as ``PoolSpec``;
     ``bytes_per_token(elem)``   bytes one token takes in one layer (``elem``: bytes of the compute
                         dtype), for sizing the pool from free memory."""
     window: Optional[int] = None
+    keep_first: int = 0
 
     def pools(self, page_size: int) -> Tuple[PoolSpec, ...]:
         raise NotImplementedError
@@ -49,6 +52,7 @@ class PagedKV(PagedSpec):
     num_kv_heads: int = 1
     head_dim: int = 0
     window: Optional[int] = None
+    keep_first: int = 0
 
     def pools(self, page_size: int) -> Tuple[PoolSpec, ...]:
         return (PoolSpec("k", (self.num_kv_heads, page_size, self.head_dim), slot_axis=1),

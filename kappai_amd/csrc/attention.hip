@@ -326,9 +326,13 @@ __global__ __launch_bounds__(64) void paged_attention_rows_kernel(
 #pragma unroll
   for (int i = 0; i < ATT_NPL; ++i) acc[i] = 0.f;
 
-  for (int base = lo; base <= pos; base += WAVE) {
-    const int tk = base + lane;
-    const bool valid = tk <= pos;
+  // the kept first positions that lie before the window, then the window: one row of places
+  const int kept = MODS ? min(mods.keep_first, lo) : 0;
+  const int n_keys = kept + pos - lo + 1;
+  for (int base = 0; base < n_keys; base += WAVE) {
+    const int place = base + lane;
+    const int tk = place < kept ? place : lo + place - kept;
+    const bool valid = place < n_keys;
     float s = -INFINITY;
     unsigned long long voff = 0;
     if (valid) {
@@ -343,7 +347,7 @@ __global__ __launch_bounds__(64) void paged_attention_rows_kernel(
     l = l * corr + wave_sum(p);
 #pragma unroll
     for (int i = 0; i < ATT_NPL; ++i) acc[i] *= corr;
-    const int nk = min(WAVE, pos - base + 1);
+    const int nk = min(WAVE, n_keys - base);
     for (int kk = 0; kk < nk; ++kk) {
       const float pk = __shfl(p, kk, WAVE);
       const unsigned lo32 = __shfl((unsigned)(voff & 0xffffffffull), kk, WAVE);
@@ -387,9 +391,10 @@ extern "C" int kappai_paged_attention_rows_scored(
     const kappai_score_mods* mods, hipStream_t stream) {
   if (T <= 0) return 0;
   if (d > MAX_HEAD_DIM || d % 8 || G < 1 || H % G || H > 65535) return (int)hipErrorInvalidValue;
-  const bool on = mods != nullptr && (mods->softcap > 0.f || mods->dist_bias || mods->sink);
-  if (on && mods->dist_bias && mods->dist_cols < 1) return (int)hipErrorInvalidValue;
-  const kappai_score_mods m = on ? *mods : kappai_score_mods{0.f, nullptr, 0, nullptr};
+  const bool on = kappai_mods_on(mods);
+  if (on && ((mods->dist_bias && mods->dist_cols < 1) || mods->keep_first < 0))
+    return (int)hipErrorInvalidValue;
+  const kappai_score_mods m = on ? *mods : kappai_score_mods{0.f, nullptr, 0, nullptr, 0};
 #define ROWS_ARGS q, q_stride, k_pool, v_pool, out, out_stride, row_pos, row_seg, block_tables, \
                   max_blocks, T, H, G, d, ps, window, scale, m, stream
   if (is_bf16) {

@@ -142,8 +142,9 @@ __device__ __forceinline__ u32x4_t load_k8(const bf16_t* __restrict__ k_pool,
 // MODS: the scores pass a cap and a bias by distance between the scaled product and the softmax
 // (score_mods.h).  The head's row of the bias table lies in LDS (tables of up to P_BIAS_MAX
 // columns; longer ones are read where they are), and a key tile that is further from every query
-// of the block than the table reaches takes the table's last column without looking.  A sink may
-// join the denominator with or without MODS.
+// of the block than the table reaches takes the table's last column without looking.  With kept
+// first positions the tiles that hold them stand in front of the window's first tile
+// (kappai_key_at).  A sink may join the denominator with or without MODS.
 #define P_BIAS_MAX 2048
 template <bool MODS>
 __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
@@ -203,7 +204,12 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
   // the diagonal take the general path.  Either way the loads of the next tile are issued
   // before the current one is worked on.
   const int lo_last = kappai_first_key(pos_last, window);
-  auto whole = [&](int kb) { return kb >= lo_last && kb + 31 <= pos_first; };
+  const int keep = MODS ? mods.keep_first : 0;
+  const int lo32 = (lo_tile / 32) * 32;
+  const int kept = MODS ? kappai_kept_places(keep, lo32) : 0;
+  auto whole = [&](int kb) {
+    return (kb >= lo_last || (MODS && kb + 31 < keep)) && kb + 31 <= pos_first;
+  };
   const int k_lane = (col % 16) * HEAD_DIM + 8 * hh;       // + 16*ks
   const int v_lane = col * ps + 4 * hh;                    // + 32*mt*ps (+ 8)
   constexpr bool P_AHEAD = HEAD_DIM <= 128;      // beyond that the registers do not suffice
@@ -238,12 +244,15 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
       }
       return;
     }
+    // what no query of the block sees reads as zero
+    const int f_lo = MODS && kb < keep ? kb : lo_tile;
+    const int f_hi = MODS && kb < lo32 ? keep - 1 : pos_last;
     const int my_key = kb + col;
     const int my_pg = col < 16 ? pg0 : pg1;
 #pragma unroll
     for (int ks = 0; ks < P_KS; ++ks)
       kfr[buf][ks] =
-          load_k8_pg(k_pool, my_pg, G, g, ps, my_key, 16 * ks + 8 * hh, lo_tile, pos_last);
+          load_k8_pg(k_pool, my_pg, G, g, ps, my_key, 16 * ks + 8 * hh, f_lo, f_hi);
 #pragma unroll
     for (int st = 0; st < 2; ++st) {
       const int key0 = kb + 16 * st + 4 * hh;
@@ -251,8 +260,8 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
 #pragma unroll
       for (int mt = 0; mt < P_MT; ++mt) {
         const int dd = 32 * mt + col;
-        vfa[buf][st][mt] = load_vt4_pg(vt_pool, pg, G, g, ps, dd, key0, lo_tile, pos_last);
-        vfb[buf][st][mt] = load_vt4_pg(vt_pool, pg, G, g, ps, dd, key0 + 8, lo_tile, pos_last);
+        vfa[buf][st][mt] = load_vt4_pg(vt_pool, pg, G, g, ps, dd, key0, f_lo, f_hi);
+        vfb[buf][st][mt] = load_vt4_pg(vt_pool, pg, G, g, ps, dd, key0 + 8, f_lo, f_hi);
       }
     }
   };
@@ -293,7 +302,7 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
 #pragma unroll
       for (int v = 0; v < 16; ++v) {
         const int key = kb + 8 * (v / 4) + 4 * hh + v % 4;
-        const bool ok = key <= my_pos && key >= my_lo;
+        const bool ok = key <= my_pos && (key >= my_lo || (MODS && key < keep));
         s[v] = ok ? s[v] : -INFINITY;
         mloc = fmaxf(mloc, s[v] * sc);
       }
@@ -332,22 +341,23 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
     }
   };
   // wave w takes the key tiles kb0 + 32 * (w + P_NW * i)
-  const int kb0 = (lo_tile / 32) * 32 + 32 * wave;
+  const int kb0 = lo32 - kept + 32 * wave;
   constexpr int KSTEP = 32 * P_NW;
+  auto at = [&](int place) { return MODS ? kappai_key_at(place, lo32, kept) : place; };
   if (P_AHEAD) {
-    if (kb0 <= pos_last) fetch(0, kb0);
+    if (kb0 <= pos_last) fetch(0, at(kb0));
     for (int kb = kb0; kb <= pos_last; kb += 2 * KSTEP) {
-      if (kb + KSTEP <= pos_last) fetch(P_NB - 1, kb + KSTEP);
-      work(0, kb);
+      if (kb + KSTEP <= pos_last) fetch(P_NB - 1, at(kb + KSTEP));
+      work(0, at(kb));
       if (kb + KSTEP <= pos_last) {
-        if (kb + 2 * KSTEP <= pos_last) fetch(0, kb + 2 * KSTEP);
-        work(P_NB - 1, kb + KSTEP);
+        if (kb + 2 * KSTEP <= pos_last) fetch(0, at(kb + 2 * KSTEP));
+        work(P_NB - 1, at(kb + KSTEP));
       }
     }
   } else {
     for (int kb = kb0; kb <= pos_last; kb += KSTEP) {
-      fetch(0, kb);
-      work(0, kb);
+      fetch(0, at(kb));
+      work(0, at(kb));
     }
   }
   if (P_NW > 1) {
@@ -923,6 +933,8 @@ __device__ __forceinline__ void qk_norm_rotate(u32x4_t (&raw)[(HEAD_DIM + 31) / 
 // of the chunks c0 = first, first + stride, ... below k_end (D_KPW keys each), with a running
 // maximum and sum per column.  Leaves the unnormalised output in o (lane: column lane % 16, d
 // rows 16 mt + 4 (lane / 16) + v), the maximum (in units of log 2) in m_run, the sum in l_run.
+// With MODS the chunks are counted in places (kappai_key_at): the kept first keys stand in front of
+// the window's, whose places are their positions.
 template <bool FUSABLE, bool MODS = false>
 __device__ __forceinline__ void attn_decode_wave(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pool,
@@ -937,9 +949,18 @@ __device__ __forceinline__ void attn_decode_wave(
   const int h = g * rep + (head_ok ? col : 0);
   // the page ids of the first chunk of keys: asked for before anything else, so that the keys
   // can be asked for as soon as they are there, whatever else is still on its way
+  const int keep = MODS ? mods->keep_first : 0;
+  const int lo32 = (lo / 32) * 32;
+  const int kept = MODS ? kappai_kept_places(keep, lo32) : 0;
   auto ask_pages = [&](int c0) {
-    const int first_page = c0 / ps;
     int my_page = -1;
+    if (MODS) {       // lane i: the page of the chunk's places 16 i .. 16 i + 15
+      const int key = kappai_key_at(c0 + 16 * lane, lo32, kept);
+      if (16 * lane < D_KPW && key / ps < max_blocks && (key <= hi || key < keep))
+        my_page = bt[key / ps];
+      return my_page;
+    }
+    const int first_page = c0 / ps;
     if (first_page + lane < max_blocks && (first_page + lane) * ps <= hi)
       my_page = bt[first_page + lane];
     return my_page;
@@ -1010,19 +1031,26 @@ __device__ __forceinline__ void attn_decode_wave(
     // kb + 8 kg .. + 7 in order, and their values are ONE 16-byte piece of a V^T row.
 #pragma unroll
     for (int c = 0; c < NCH; ++c) {
-      const int kb = c0 + 32 * c;
+      const int kb = MODS ? kappai_key_at(c0 + 32 * c, lo32, kept) : c0 + 32 * c;
+      // (what the row does not see reads as zero)
+      const int f_lo = MODS && kb < keep ? kb : lo, f_hi = MODS && kb < lo32 ? keep - 1 : hi;
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt) {
         const int key = kb + 8 * (col / 4) + 4 * tt + col % 4;
-        const int page = __shfl(my_page, min(key / ps - first_page, WAVE - 1), WAVE);
+        const int page =
+            MODS ? __shfl(my_page, 2 * c + (key - kb) / 16, WAVE)
+                 : __shfl(my_page, min(key / ps - first_page, WAVE - 1), WAVE);
 #pragma unroll
         for (int ks = 0; ks < D_KS; ++ks)
-          ch.kf[c][tt][ks] = load_k8_pg(k_pool, page, G, g, ps, key, 32 * ks + 8 * kg, lo, hi);
+          ch.kf[c][tt][ks] = load_k8_pg(k_pool, page, G, g, ps, key, 32 * ks + 8 * kg, f_lo, f_hi);
       }
-      const int pv = __shfl(my_page, min((kb + 8 * kg) / ps - first_page, WAVE - 1), WAVE);
+      const int pv =
+          MODS ? __shfl(my_page, 2 * c + kg / 2, WAVE)
+               : __shfl(my_page, min((kb + 8 * kg) / ps - first_page, WAVE - 1), WAVE);
 #pragma unroll
       for (int mt = 0; mt < D_MT; ++mt)
-        ch.vv[c][mt] = load_vt8_pg(vt_pool, pv, G, g, ps, 16 * mt + col, kb + 8 * kg, lo, hi);
+        ch.vv[c][mt] = load_vt8_pg(vt_pool, pv, G, g, ps, 16 * mt + col, kb + 8 * kg,
+                                    f_lo, f_hi);
     }
   };
   // the pools do not hold the row's own key and value yet (or only just): the chunk that holds
@@ -1057,8 +1085,8 @@ __device__ __forceinline__ void attn_decode_wave(
   auto work = [&](int c0, const Chunk& ch) {
 #pragma unroll
     for (int c = 0; c < NCH; ++c) {
-      const int kb = c0 + 32 * c;
-      if (kb >= k_end) break;
+      if (c0 + 32 * c >= k_end) break;
+      const int kb = MODS ? kappai_key_at(c0 + 32 * c, lo32, kept) : c0 + 32 * c;
       f32x4_t s[2];
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt) {
@@ -1075,7 +1103,7 @@ __device__ __forceinline__ void attn_decode_wave(
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
           const int key = kb + 8 * kg + 4 * tt + v;
-          const bool ok = key >= lo && key <= hi;
+          const bool ok = (key >= lo || (MODS && key < keep)) && key <= hi;
           if (MODS) {
             float x = s[tt][v] * scale;
             if (mods->softcap > 0.f) x = kappai_fast_cap(x, mods->softcap);
@@ -1157,17 +1185,18 @@ __device__ __forceinline__ void attn_decode_wave(
 // no fewer than the longest row needs to fit into n_splits.  Every wave of the step computes the
 // same number from the same table; splits past a row's keys do nothing and are not merged.
 #define D_TARGET_WAVES 2048
-__device__ __forceinline__ int keys_of_row(int pos, int window) {
-  const int lo = kappai_first_key(pos, window);
-  return pos + 1 - (lo / 32) * 32;
+__device__ __forceinline__ int keys_of_row(int pos, int window, int keep) {
+  const int lo32 = kappai_first_key(pos, window) / 32 * 32;
+  return pos + 1 - lo32 + kappai_kept_places(keep, lo32);
 }
 __device__ __forceinline__ int step_keys_per_split(const int* __restrict__ row_pos,
                                                    const int* __restrict__ row_ids, int n_rows,
-                                                   int window, int G, int kps_min, int n_splits) {
+                                                   int window, int keep, int G, int kps_min,
+                                                   int n_splits) {
   const int lane = threadIdx.x % WAVE;
   int total32 = 0, longest = 0;                  // the sum in units of 32 keys, rounded up by row
   for (int i = lane; i < n_rows; i += WAVE) {
-    const int n = keys_of_row(row_pos[row_ids ? row_ids[i] : i], window);
+    const int n = keys_of_row(row_pos[row_ids ? row_ids[i] : i], window, keep);
     total32 += (n + 31) / 32;
     longest = max(longest, n);
   }
@@ -1208,12 +1237,14 @@ __global__ __launch_bounds__(64) void attn_decode_kernel(
   const int col = lane % 16, kg = lane / 16;
   const int pos = row_pos[t];
   const int seg = row_seg[t];
-  const int kps = PLAN ? step_keys_per_split(row_pos, row_ids, (int)gridDim.x, window, G,
+  const int keep = MODS ? mods.keep_first : 0;
+  const int kps = PLAN ? step_keys_per_split(row_pos, row_ids, (int)gridDim.x, window, keep, G,
                                              keys_per_split, n_splits)
                        : keys_per_split;
   const int* bt = block_tables + (size_t)seg * max_blocks;
   const int lo = kappai_first_key(pos, window);
-  const int k_begin = (lo / 32) * 32 + split * kps;
+  const int lo32 = (lo / 32) * 32;
+  const int k_begin = lo32 - (MODS ? kappai_kept_places(keep, lo32) : 0) + split * kps;
   if (k_begin > pos) return;                                   // a split past the row's keys
   const int k_end = min(k_begin + kps, pos + 1);                // exclusive
   const bool head_ok = col < rep;
@@ -1259,7 +1290,8 @@ __global__ __launch_bounds__(D_BLOCK_MAX_WAVES * WAVE) void attn_decode_block_ke
   const int pos = row_pos[t];
   const int* bt = block_tables + (size_t)row_seg[t] * max_blocks;
   const int lo = kappai_first_key(pos, window);
-  const int k_begin = (lo / 32) * 32;
+  const int lo32 = (lo / 32) * 32;
+  const int k_begin = lo32 - (MODS ? kappai_kept_places(mods.keep_first, lo32) : 0);
   const int k_end = pos + 1;
   f32x4_t o[D_MT];
   float m_run, l_run;
@@ -1310,7 +1342,7 @@ __global__ __launch_bounds__(D_BLOCK_MAX_WAVES * WAVE) void attn_decode_block_ke
 __global__ __launch_bounds__(MERGE_WAVES * WAVE) void attn_merge_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     bf16_t* __restrict__ out, int out_stride, int H, int splits_stride,
-    const int* __restrict__ row_ids, const int* __restrict__ row_pos, int window, int G,
+    const int* __restrict__ row_ids, const int* __restrict__ row_pos, int window, int keep, int G,
     int kps_min, int planned, const float* __restrict__ sink) {
   constexpr int NPL = (HEAD_DIM + WAVE - 1) / WAVE;
   __shared__ float sh_acc[MERGE_WAVES][NPL * WAVE];
@@ -1341,10 +1373,10 @@ __global__ __launch_bounds__(MERGE_WAVES * WAVE) void attn_merge_kernel(
   if (wave + MERGE_WAVES * lane < splits_stride)
     ml_first = *reinterpret_cast<const float2*>(part_ml + 2 * (base + wave + MERGE_WAVES * lane));
   // the splits of this row that had keys (the decode kernel's own rule)
-  const int kps = planned ? step_keys_per_split(row_pos, row_ids, (int)gridDim.x, window, G,
+  const int kps = planned ? step_keys_per_split(row_pos, row_ids, (int)gridDim.x, window, keep, G,
                                                 kps_min, splits_stride)
                           : kps_min;
-  const int n_splits = (keys_of_row(row_pos[t], window) + kps - 1) / kps;
+  const int n_splits = (keys_of_row(row_pos[t], window, keep) + kps - 1) / kps;
 #pragma unroll
   for (int k = 0; k < MERGE_AHEAD; ++k)
 #pragma unroll
@@ -1424,6 +1456,9 @@ extern "C" int kappai_attn_decode_block_scored(const void* q, int q_stride, cons
   if (ps % 16 || G < 1 || H % G || H / G > 16 || G > 65535 || (q_stride % 8) || n_waves < 1 ||
       n_waves > kappai_attn_decode_block_waves(H / G))
     return (int)hipErrorInvalidValue;
+  if (kappai_mods_change_scores(mods) &&
+      (mods->keep_first < 0 || (mods->dist_bias != nullptr && mods->dist_cols < 1)))
+    return (int)hipErrorInvalidValue;
   const int rep = H / G;
   const size_t lds = (size_t)n_waves * (rep * HEAD_DIM + 32) * sizeof(float);
   if (kappai_mods_change_scores(mods))
@@ -1436,7 +1471,7 @@ extern "C" int kappai_attn_decode_block_scored(const void* q, int q_stride, cons
                        stream, (const bf16_t*)q, q_stride, (const bf16_t*)k_pool,
                        (const bf16_t*)vt_pool, (bf16_t*)out, out_stride, row_pos, row_seg,
                        block_tables, max_blocks, H, G, ps, window, scale,
-                       kappai_score_mods{0.f, nullptr, 0, mods != nullptr ? mods->sink : nullptr});
+                       kappai_score_mods{0.f, nullptr, 0, mods != nullptr ? mods->sink : nullptr, 0});
   KAPPAI_RETURN_LAUNCH_STATUS();
 }
 
@@ -1485,7 +1520,8 @@ extern "C" int kappai_attn_prefill_scored(const void* q, int q_stride, const voi
   const float* sink = mods != nullptr ? mods->sink : nullptr;
   if (kappai_mods_change_scores(mods)) {
     if (ps % 16 || G < 1 || H % G || H > 65535 || (q_stride % 8) || (out_stride % 4) ||
-        variant == 2 || (mods->dist_bias != nullptr && mods->dist_cols < 1))
+        variant == 2 || mods->keep_first < 0 ||
+        (mods->dist_bias != nullptr && mods->dist_cols < 1))
       return (int)hipErrorInvalidValue;
     hipLaunchKernelGGL(attn_prefill_kernel<true>, dim3(n_tiles, H), dim3(P_NW * WAVE), 0, stream,
                        (const bf16_t*)q, q_stride, (const bf16_t*)k_pool, (const bf16_t*)vt_pool,
@@ -1515,7 +1551,7 @@ extern "C" int kappai_attn_prefill_scored(const void* q, int q_stride, const voi
   hipLaunchKernelGGL(attn_prefill_kernel<false>, dim3(n_tiles, H), dim3(P_NW * WAVE), 0, stream,
                      (const bf16_t*)q, q_stride, (const bf16_t*)k_pool, (const bf16_t*)vt_pool,
                      (bf16_t*)out, out_stride, q_tiles, row_pos, block_tables, max_blocks, H, G,
-                     ps, window, scale, kappai_score_mods{0.f, nullptr, 0, sink});
+                     ps, window, scale, kappai_score_mods{0.f, nullptr, 0, sink, 0});
   KAPPAI_RETURN_LAUNCH_STATUS();
 }
 
@@ -1537,9 +1573,11 @@ static int launch_decode(const void* q, int q_stride, const void* k_pool, const 
                          hipStream_t stream, const kappai_score_mods* mods = nullptr) {
   if (T <= 0) return 0;
   const bool scored = kappai_mods_change_scores(mods);
-  if (scored && qk.on) return (int)hipErrorInvalidValue;
+  if (scored && (qk.on || mods->keep_first < 0 ||
+                 (mods->dist_bias != nullptr && mods->dist_cols < 1)))
+    return (int)hipErrorInvalidValue;
   const kappai_score_mods m =
-      scored ? *mods : kappai_score_mods{0.f, nullptr, 0, mods != nullptr ? mods->sink : nullptr};
+      scored ? *mods : kappai_score_mods{0.f, nullptr, 0, mods != nullptr ? mods->sink : nullptr, 0};
   if (ps % 16 || G < 1 || H % G || H / G > 16 || G > 65535 || n_splits < 1 || n_splits > 65535 ||
       keys_per_split < D_KPW || keys_per_split % D_KPW || (q_stride % 8))
     return (int)hipErrorInvalidValue;
@@ -1561,7 +1599,8 @@ static int launch_decode(const void* q, int q_stride, const void* k_pool, const 
 #undef KAPPAI_DECODE
   hipLaunchKernelGGL(attn_merge_kernel, dim3(T, H), dim3(MERGE_WAVES * WAVE), 0, stream,
                      (const float*)part_o, (const float*)part_ml, (bf16_t*)out, out_stride, H,
-                     n_splits, row_ids, row_pos, window, G, keys_per_split, plan ? 1 : 0, m.sink);
+                     n_splits, row_ids, row_pos, window, m.keep_first, G, keys_per_split, plan ? 1 : 0,
+                     m.sink);
   KAPPAI_RETURN_LAUNCH_STATUS();
 }
 

@@ -13,7 +13,8 @@
 //                           the keys' up-projection fills (headwise_linear)
 //   headwise_linear         y[t, h, :] = W[h] x[t, h, :], a matrix per head
 //   head_norm_rotate_store  RMS norm of every q and k head by itself (one weight [d] for all
-//                           heads), rotation of the first places, heads of d and dv widened to D
+//                           heads), rotation of the first places, heads of d and dv widened to D;
+//                           the values may be the keys as projected
 #include "common.h"
 
 #define AP_THREADS 256
@@ -400,8 +401,9 @@ extern "C" int kappai_rotate_widen_store(
 // head_norm_rotate_store: grouped-query heads whose queries and keys (d) and values (dv) differ
 // in size.  Every q and k head is divided by the root mean square of its own d places and
 // multiplied by a weight [d] that all heads share (q_norm_w / k_norm_w; null: no norm); then the
-// first rot_dims places of the head turn by the row's position.  proj [T, H d + G d + G dv].
-// Queries leave as H heads of D (zeros behind d); keys and values go to the pools as G heads of
+// first rot_dims places of the head turn by the row's position.  proj [T, H d + G d + G dv]; with
+// `v_at` = H d (dv = d) there are no value columns and a kv head's value is its key as projected,
+// before norm and rotation (v_at: the column at which the values start).  Queries leave as H heads of D (zeros behind d); keys and values go to the pools as G heads of
 // D.  A wave a head: the sum of squares stays in the wave; a block takes four heads of a row
 // (grid: rows x groups of four heads).
 // ---------------------------------------------------------------------------------------
@@ -412,12 +414,12 @@ __global__ __launch_bounds__(AP_THREADS) void head_norm_rotate_store_kernel(
     const float* __restrict__ sin_tab, int rot_dims, int rot_mode, T* __restrict__ k_pool,
     T* __restrict__ v_pool, const int* __restrict__ row_pos, const int* __restrict__ row_seg,
     const int* __restrict__ block_tables, int max_blocks, int H, int G, int d, int dv, int D,
-    int ps, T* __restrict__ q_out) {
+    int ps, int v_at, T* __restrict__ q_out) {
   const int t = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   constexpr int NW = AP_THREADS / WAVE;
   const int pos = row_pos[t];
   const T* row = proj + (size_t)t * stride;
-  const int nq = H * d, nk = G * d, half = rot_dims / 2;
+  const int nq = H * d, half = rot_dims / 2;
   const float* ct = cos_tab + (size_t)pos * half;
   const float* st = sin_tab + (size_t)pos * half;
   size_t page = 0;
@@ -430,7 +432,7 @@ __global__ __launch_bounds__(AP_THREADS) void head_norm_rotate_store_kernel(
       const int g = head - H - G;
       for (int e = lane; e < D; e += WAVE)
         from_f32(v_pool + ((page * G + g) * D + e) * ps + slot,
-                 e < dv ? to_f32(row[nq + nk + g * dv + e]) : 0.f);
+                 e < dv ? to_f32(row[v_at + g * dv + e]) : 0.f);
       continue;
     }
     const bool is_q = head < H;
@@ -479,7 +481,7 @@ __global__ __launch_bounds__(AP_THREADS) void head_norm_rotate_store_vec_kernel(
     const float* __restrict__ sin_tab, int rot_dims, bf16_t* __restrict__ k_pool,
     bf16_t* __restrict__ v_pool, const int* __restrict__ row_pos, const int* __restrict__ row_seg,
     const int* __restrict__ block_tables, int max_blocks, int H, int G, int d, int dv, int D,
-    int ps, bf16_t* __restrict__ q_out) {
+    int ps, int v_at, bf16_t* __restrict__ q_out) {
   constexpr int HPW = WAVE / LPH, NW = AP_THREADS / WAVE;
   const int t = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int head = (blockIdx.y * NW + wave) * HPW + lane / LPH, sub = lane % LPH, e0 = sub * 8;
@@ -487,14 +489,14 @@ __global__ __launch_bounds__(AP_THREADS) void head_norm_rotate_store_vec_kernel(
   const bool live = head < n_heads && e0 < D && (head < H || k_pool != nullptr);
   const int pos = row_pos[t];
   const bf16_t* row = proj + (size_t)t * stride;
-  const int nq = H * d, nk = G * d, half = rot_dims / 2;
+  const int nq = H * d, half = rot_dims / 2;
   const bool is_v = head >= H + G, is_q = head < H;
   const int width = is_v ? dv : d;
   float v[8];
 #pragma unroll
   for (int i = 0; i < 8; ++i) v[i] = 0.f;
   if (live && e0 < width) {
-    const bf16_t* src = is_q ? row + head * d : is_v ? row + nq + nk + (head - H - G) * dv
+    const bf16_t* src = is_q ? row + head * d : is_v ? row + v_at + (head - H - G) * dv
                                                      : row + nq + (head - H) * d;
     load8(src + e0, v);
   }
@@ -546,14 +548,15 @@ extern "C" int kappai_head_norm_rotate_store(
     const void* proj, int stride, const float* q_norm_w, const float* k_norm_w, float eps,
     const float* cos_tab, const float* sin_tab, int rot_dims, int rot_mode, void* k_pool,
     void* v_pool, const int* row_pos, const int* row_seg, const int* block_tables, int max_blocks,
-    int T, int H, int G, int d, int dv, int D, int ps, void* q_out, int is_bf16,
+    int T, int H, int G, int d, int dv, int D, int ps, int values_are_keys, void* q_out, int is_bf16,
     hipStream_t stream) {
   if (T <= 0) return 0;
   if (H < 1 || G < 1 || d < 1 || dv < 1 || D < d || D < dv || ps < 1 || rot_dims < 0 ||
-      rot_dims > d || rot_dims % 2 || rot_mode < 0 || rot_mode > 2 ||
+      rot_dims > d || rot_dims % 2 || (values_are_keys && dv != d) || rot_mode < 0 || rot_mode > 2 ||
       (rot_mode && rot_dims && (!cos_tab || !sin_tab)))
     return (int)hipErrorInvalidValue;
   if (rot_dims == 0) rot_mode = 0;
+  const int v_at = values_are_keys ? H * d : (H + G) * d;
   const int lph = D / 8, half = rot_dims / 2;
   if (is_bf16 && d % 8 == 0 && dv % 8 == 0 && D % 8 == 0 && stride % 8 == 0 &&
       (uintptr_t)proj % 16 == 0 && (uintptr_t)q_out % 16 == 0 && (uintptr_t)k_pool % 16 == 0 &&
@@ -568,7 +571,7 @@ extern "C" int kappai_head_norm_rotate_store(
   hipLaunchKernelGGL(head_norm_rotate_store_vec_kernel<L>, grid, dim3(AP_THREADS), 0, stream,     \
                      (const bf16_t*)proj, stride, q_norm_w, k_norm_w, eps, cos_tab, sin_tab,      \
                      rot_mode ? rot_dims : 0, (bf16_t*)k_pool, (bf16_t*)v_pool, row_pos, row_seg, \
-                     block_tables, max_blocks, H, G, d, dv, D, ps, (bf16_t*)q_out)
+                     block_tables, max_blocks, H, G, d, dv, D, ps, v_at, (bf16_t*)q_out)
     switch (lph) {
       case 1: HNRS_VEC(1); break;
       case 2: HNRS_VEC(2); break;
@@ -585,11 +588,11 @@ extern "C" int kappai_head_norm_rotate_store(
     hipLaunchKernelGGL(head_norm_rotate_store_kernel<bf16_t>, hn_grid, dim3(AP_THREADS), 0,
                        stream, (const bf16_t*)proj, stride, q_norm_w, k_norm_w, eps, cos_tab,
                        sin_tab, rot_dims, rot_mode, (bf16_t*)k_pool, (bf16_t*)v_pool, row_pos,
-                       row_seg, block_tables, max_blocks, H, G, d, dv, D, ps, (bf16_t*)q_out);
+                       row_seg, block_tables, max_blocks, H, G, d, dv, D, ps, v_at, (bf16_t*)q_out);
   else
     hipLaunchKernelGGL(head_norm_rotate_store_kernel<float>, hn_grid, dim3(AP_THREADS), 0, stream,
                        (const float*)proj, stride, q_norm_w, k_norm_w, eps, cos_tab, sin_tab,
                        rot_dims, rot_mode, (float*)k_pool, (float*)v_pool, row_pos, row_seg,
-                       block_tables, max_blocks, H, G, d, dv, D, ps, (float*)q_out);
+                       block_tables, max_blocks, H, G, d, dv, D, ps, v_at, (float*)q_out);
   KAPPAI_RETURN_LAUNCH_STATUS();
 }

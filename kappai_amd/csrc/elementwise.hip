@@ -9,11 +9,11 @@
 // ---------------------------------------------------------------------------------------
 template <typename TW>
 __global__ void embed_rows_kernel(const int* __restrict__ ids, const TW* __restrict__ table,
-                                  float* __restrict__ out, int D) {
+                                  float* __restrict__ out, int D, float scale) {
   const int t = blockIdx.x;
   const TW* src = table + (size_t)ids[t] * D;
   float* dst = out + (size_t)t * D;
-  for (int i = threadIdx.x; i < D; i += blockDim.x) dst[i] = to_f32(src[i]);
+  for (int i = threadIdx.x; i < D; i += blockDim.x) dst[i] = to_f32(src[i]) * scale;
 }
 
 // The same from a bfloat16 table that is kept in the order of the matrix cores' fragments (a
@@ -21,7 +21,7 @@ __global__ void embed_rows_kernel(const int* __restrict__ ids, const TW* __restr
 // lane = (column % 32) / 8 * 16 + row % 16); D a multiple of 32.
 __global__ void embed_rows_fragments_kernel(const int* __restrict__ ids,
                                             const bf16_t* __restrict__ table,
-                                            float* __restrict__ out, int D) {
+                                            float* __restrict__ out, int D, float scale) {
   const int t = blockIdx.x;
   const size_t r = (size_t)ids[t];
   const bf16_t* src = table + (r / 16) * 16 * D + (r % 16) * 8;
@@ -35,27 +35,36 @@ __global__ void embed_rows_fragments_kernel(const int* __restrict__ ids,
     lo.z = __uint_as_float(u[1] << 16), lo.w = __uint_as_float(u[1] & 0xffff0000u);
     hi.x = __uint_as_float(u[2] << 16), hi.y = __uint_as_float(u[2] & 0xffff0000u);
     hi.z = __uint_as_float(u[3] << 16), hi.w = __uint_as_float(u[3] & 0xffff0000u);
+    lo.x *= scale, lo.y *= scale, lo.z *= scale, lo.w *= scale;
+    hi.x *= scale, hi.y *= scale, hi.z *= scale, hi.w *= scale;
     *reinterpret_cast<float4*>(dst + 8 * c) = lo;
     *reinterpret_cast<float4*>(dst + 8 * c + 4) = hi;
   }
 }
 
-// table_is_bf16: 0 = float32 rows, 1 = bfloat16 rows, 2 = bfloat16 in fragment order
-extern "C" int kappai_embed_rows(const int* ids, const void* table, int table_is_bf16, float* out,
-                                 int T, int D, hipStream_t stream) {
+// table_is_bf16: 0 = float32 rows, 1 = bfloat16 rows, 2 = bfloat16 in fragment order; `scale`: a
+// factor on every row
+extern "C" int kappai_embed_rows_scaled(const int* ids, const void* table, int table_is_bf16,
+                                        float* out, int T, int D, float scale,
+                                        hipStream_t stream) {
   if (T <= 0) return 0;
   const int threads = D >= 1024 ? 256 : (D >= 256 ? 128 : 64);
   if (table_is_bf16 == 2) {
     if (D % 32 || ((uintptr_t)table % 16) || ((uintptr_t)out % 16)) return (int)hipErrorInvalidValue;
     hipLaunchKernelGGL(embed_rows_fragments_kernel, dim3(T), dim3(threads), 0, stream, ids,
-                       (const bf16_t*)table, out, D);
+                       (const bf16_t*)table, out, D, scale);
   } else if (table_is_bf16)
     hipLaunchKernelGGL(embed_rows_kernel<bf16_t>, dim3(T), dim3(threads), 0, stream, ids,
-                       (const bf16_t*)table, out, D);
+                       (const bf16_t*)table, out, D, scale);
   else
     hipLaunchKernelGGL(embed_rows_kernel<float>, dim3(T), dim3(threads), 0, stream, ids,
-                       (const float*)table, out, D);
+                       (const float*)table, out, D, scale);
   KAPPAI_RETURN_LAUNCH_STATUS();
+}
+
+extern "C" int kappai_embed_rows(const int* ids, const void* table, int table_is_bf16, float* out,
+                                 int T, int D, hipStream_t stream) {
+  return kappai_embed_rows_scaled(ids, table, table_is_bf16, out, T, D, 1.0f, stream);
 }
 
 // ---------------------------------------------------------------------------------------
@@ -150,6 +159,152 @@ extern "C" int kappai_output_norm_add(const void* a, int a_is_bf16, int a_parts,
     if (rows_is_bf16) KAPPAI_OUT_NORM(float, bf16_t); else KAPPAI_OUT_NORM(float, float);
   }
 #undef KAPPAI_OUT_NORM
+  KAPPAI_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------------
+// Pointwise norms that saturate, n(x) = tanh(alpha x) w + b (one alpha a row, w and b [D]), on both
+// sides of a sublayer in one pass over the stream: resid += n_post(y), rows = n_pre(resid).  No place
+// looks at another, so there is nothing to sum and a thread works on its own VEC columns from the
+// loads to the store.  y comes as
+//   TY rows, or float planes [parts][T][D] that are added in order (a product cut over its input
+//   dimension), or, with slot_of_pair, as a mixture's experts left it: the sum over the row's `top`
+//   choices of wts[t, k] * y[slot of (t, k)], in the order of k.
+// post.w null: y is added as it is; pre.w null: no rows are wanted.  `pick`: only these rows are
+// normalised, and the stream keeps its old values.  Everything in float32.
+// ---------------------------------------------------------------------------------------
+struct kappai_tanh_norm {
+  float alpha;
+  const float* w;
+  const float* b;
+};
+
+template <int VEC>
+__device__ __forceinline__ void load_cols(const float* p, float (&v)[VEC]) {
+  if (VEC == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    v[0] = a.x; v[VEC > 1 ? 1 : 0] = a.y; v[VEC > 2 ? 2 : 0] = a.z; v[VEC > 3 ? 3 : 0] = a.w;
+  } else {
+    v[0] = p[0];
+  }
+}
+template <int VEC>
+__device__ __forceinline__ void load_cols(const bf16_t* p, float (&v)[VEC]) {
+  if (VEC == 4) {
+    const uint2 a = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(a.x << 16); v[VEC > 1 ? 1 : 0] = __uint_as_float(a.x & 0xffff0000u);
+    v[VEC > 2 ? 2 : 0] = __uint_as_float(a.y << 16);
+    v[VEC > 3 ? 3 : 0] = __uint_as_float(a.y & 0xffff0000u);
+  } else {
+    v[0] = to_f32(p[0]);
+  }
+}
+template <int VEC>
+__device__ __forceinline__ void store_cols(float* p, const float (&v)[VEC]) {
+  if (VEC == 4)
+    *reinterpret_cast<float4*>(p) =
+        make_float4(v[0], v[VEC > 1 ? 1 : 0], v[VEC > 2 ? 2 : 0], v[VEC > 3 ? 3 : 0]);
+  else
+    p[0] = v[0];
+}
+template <int VEC>
+__device__ __forceinline__ void store_cols(bf16_t* p, const float (&v)[VEC]) {
+  if (VEC == 4)
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v[0], v[VEC > 1 ? 1 : 0]),
+                                              pack_bf16x2(v[VEC > 2 ? 2 : 0], v[VEC > 3 ? 3 : 0]));
+  else
+    from_f32(p, v[0]);
+}
+
+template <typename TY, typename TO, int VEC>
+__global__ __launch_bounds__(256) void tanh_norm_kernel(
+    float* __restrict__ resid, const TY* __restrict__ y, int parts, size_t plane,
+    const int* __restrict__ slot_of_pair, const float* __restrict__ wts, int top,
+    kappai_tanh_norm post, kappai_tanh_norm pre, const int* __restrict__ pick, long n_pieces,
+    int D, int store, TO* __restrict__ rows) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n_pieces) return;
+  const int per_row = D / VEC;
+  const long r = i / per_row;
+  const int c = (int)(i - r * per_row) * VEC;
+  const size_t t = pick != nullptr ? (size_t)pick[r] : (size_t)r;
+  float x[VEC];
+  load_cols<VEC>(resid + t * D + c, x);
+  if (y != nullptr) {
+    float u[VEC], w[VEC], b[VEC];
+    if (slot_of_pair != nullptr) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) u[j] = 0.f;
+#pragma unroll 4
+      for (int k = 0; k < top; ++k) {
+        float v[VEC];
+        load_cols<VEC>(y + (size_t)slot_of_pair[t * top + k] * D + c, v);
+        const float f = wts[t * top + k];
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) u[j] = fmaf(f, v[j], u[j]);
+      }
+    } else {
+      load_cols<VEC>(y + t * D + c, u);
+#pragma unroll 4
+      for (int k = 1; k < parts; ++k) {
+        float v[VEC];
+        load_cols<VEC>(y + k * plane + t * D + c, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) u[j] += v[j];
+      }
+    }
+    if (post.w != nullptr) {
+      load_cols<VEC>(post.w + c, w);
+      load_cols<VEC>(post.b + c, b);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) u[j] = fmaf(tanhf(post.alpha * u[j]), w[j], b[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[j] += u[j];
+    if (store) store_cols<VEC>(resid + t * D + c, x);
+  }
+  if (rows == nullptr) return;
+  float w[VEC], b[VEC];
+  load_cols<VEC>(pre.w + c, w);
+  load_cols<VEC>(pre.b + c, b);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) x[j] = fmaf(tanhf(pre.alpha * x[j]), w[j], b[j]);
+  store_cols<VEC>(rows + r * D + c, x);
+}
+
+extern "C" int kappai_tanh_norm_step(float* resid, const void* y, int y_is_bf16, int parts,
+                                     const int* slot_of_pair, const float* wts, int top,
+                                     float post_alpha, const float* post_w, const float* post_b,
+                                     float pre_alpha, const float* pre_w, const float* pre_b,
+                                     const int* pick, int n_rows, int T, int D, void* rows,
+                                     int rows_is_bf16, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (D < 1 || (y && parts < 1) || (y_is_bf16 && (parts != 1 || slot_of_pair)) ||
+      (slot_of_pair && (!y || !wts || top < 1)) || (post_w && !post_b) ||
+      (rows && (!pre_w || !pre_b)) || (!pick && n_rows != T))
+    return (int)hipErrorInvalidValue;
+  const bool vec = D % 4 == 0 &&
+                   ((uintptr_t)resid | (uintptr_t)y | (uintptr_t)post_w | (uintptr_t)post_b |
+                    (uintptr_t)pre_w | (uintptr_t)pre_b | (uintptr_t)rows) % 16 == 0;
+  const long pieces = (long)n_rows * (vec ? D / 4 : D);
+  // few rows: blocks of one wave, so that the pieces spread over the chip
+  const int threads = pieces <= 64 * 1024 ? 64 : 256;
+  const long blocks = (pieces + threads - 1) / threads;
+  if (blocks > 0x7fffffffL) return (int)hipErrorInvalidValue;
+  const kappai_tanh_norm post{post_alpha, post_w, post_b}, pre{pre_alpha, pre_w, pre_b};
+#define KAPPAI_TANH_NORM(TY, TO, V)                                                              \
+  hipLaunchKernelGGL((tanh_norm_kernel<TY, TO, V>), dim3((unsigned)blocks), dim3(threads), 0,    \
+                     stream, resid, (const TY*)y, parts, (size_t)T * D, slot_of_pair, wts, top,  \
+                     post, pre, pick, pieces, D, pick ? 0 : 1, (TO*)rows)
+#define KAPPAI_TANH_NORM_V(TY, TO)                                                               \
+  if (vec) KAPPAI_TANH_NORM(TY, TO, 4); else KAPPAI_TANH_NORM(TY, TO, 1)
+  if (y_is_bf16) {
+    if (rows_is_bf16) { KAPPAI_TANH_NORM_V(bf16_t, bf16_t); } else { KAPPAI_TANH_NORM_V(bf16_t, float); }
+  } else {
+    if (rows_is_bf16) { KAPPAI_TANH_NORM_V(float, bf16_t); } else { KAPPAI_TANH_NORM_V(float, float); }
+  }
+#undef KAPPAI_TANH_NORM_V
+#undef KAPPAI_TANH_NORM
   KAPPAI_RETURN_LAUNCH_STATUS();
 }
 

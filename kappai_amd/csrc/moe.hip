@@ -2,7 +2,8 @@
 // order, and the weighted sum.  Nothing is read back by the host: every launch is sized by the
 // number of rows alone, so a step with experts can be captured in a graph.
 //   moe_route     z = W_router h in float32, the `top` largest chosen (lowest index on ties),
-//                 weights = softmax over the chosen logits
+//                 weights = softmax over the chosen logits; or scores s = sigmoid(z), the choice by
+//                 s + a correction within the best groups of experts, weights = s times a constant
 //   moe_plan      (row, choice) pairs in expert order, every expert's run starting on a tile of
 //                 MOE_TILE_M slots: slot_of_pair, pair_of_slot (-1: empty), tile_expert (-1: unused)
 //   moe_gemm      tile by tile: act = silu(x Wg^T) * (x Wu^T) on gathered rows, or y = act Wd^T
@@ -20,15 +21,64 @@ extern "C" int kappai_moe_tile_rows() { return MOE_TILE_M; }
 
 #define MOE_ROUTE_GROUP 16      // experts whose sums a thread carries side by side
 
+// How a router that squashes every logit by itself chooses: score s = sigmoid(z), choice score
+// s + correction[e] (null: s).  The experts form `groups` equal groups of neighbours; a group's
+// score is the sum of its two largest choice scores, and only experts of the `keep` best groups can
+// be chosen (groups 1: all of them).  The weight of a chosen expert is s * scale.
+struct moe_squashed_choice {
+  const float* correction;
+  int groups, keep;
+  float scale;
+};
+
+// The choice scores of the row in `choice` [E] (logits on entry) and the scores in `score` [E]; one
+// wave.  `group_score`: LDS for `groups` floats.
+__device__ __forceinline__ void moe_squash(const moe_squashed_choice& c, int E, float* choice,
+                                           float* score, float* group_score) {
+  const int lane = threadIdx.x % WAVE;
+  auto meet = [] {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  };
+  for (int e = lane; e < E; e += WAVE) {
+    const float s = 1.0f / (1.0f + expf(-choice[e]));
+    score[e] = s;
+    choice[e] = c.correction ? s + c.correction[e] : s;
+  }
+  meet();
+  if (c.groups <= 1 || c.keep >= c.groups) return;
+  const int size = E / c.groups;
+  for (int g = lane; g < c.groups; g += WAVE) {
+    float a = -INFINITY, b = -INFINITY;           // the two largest
+    for (int e = g * size; e < (g + 1) * size; ++e) {
+      const float v = choice[e];
+      b = fmaxf(b, fminf(a, v));
+      a = fmaxf(a, v);
+    }
+    group_score[g] = size > 1 ? a + b : a;
+  }
+  meet();
+  for (int g = lane; g < c.groups; g += WAVE) {
+    const float mine = group_score[g];
+    int better = 0;
+    for (int o = 0; o < c.groups; ++o)
+      better += group_score[o] > mine || (group_score[o] == mine && o < g) ? 1 : 0;
+    if (better >= c.keep)
+      for (int e = g * size; e < (g + 1) * size; ++e) choice[e] = -INFINITY;
+  }
+  meet();
+}
+
 // A block a row.  The threads stride over the row four columns at a time (one column at a time
 // when the width or an address does not allow 16-byte loads), each with the sums of a group of
 // experts, whose loads are all asked for before the first is used; the waves' sums meet in LDS
 // and are added in the order of the waves.  Then the first wave chooses.
-template <typename T, int VEC>
+template <typename T, int VEC, bool SQUASHED>
 __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
     const T* __restrict__ x, int ldx, const float* __restrict__ router,
-    const float* __restrict__ bias, int n_rows, int D, int E, int top, int* __restrict__ idx,
-    float* __restrict__ wts) {
+    const float* __restrict__ bias, int n_rows, int D, int E, int top, moe_squashed_choice sq,
+    int* __restrict__ idx, float* __restrict__ wts) {
   extern __shared__ float route_lds[];
   constexpr int NW = MOE_THREADS / WAVE;
   float* logits = route_lds;                       // [E]
@@ -74,6 +124,8 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
     __syncthreads();
   }
   if (wave != 0) return;
+  float* score = part + MOE_ROUTE_GROUP * NW;      // [E], then [groups] (squashed scores only)
+  if (SQUASHED) moe_squash(sq, E, logits, score, score + E);
   float cv[MOE_MAX_TOP];
   int ci[MOE_MAX_TOP];
 #pragma unroll
@@ -96,6 +148,16 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
     }
   }
   if (lane == 0) {
+    if (SQUASHED) {
+#pragma unroll
+      for (int k = 0; k < MOE_MAX_TOP; ++k)
+        if (k < top) {
+          const int e = ci[k] < E ? ci[k] : 0;
+          idx[(size_t)row * top + k] = e;
+          wts[(size_t)row * top + k] = score[e] * sq.scale;
+        }
+      return;
+    }
     float sum = 0.f;
 #pragma unroll
     for (int k = 0; k < MOE_MAX_TOP; ++k)
@@ -109,23 +171,46 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
   }
 }
 
+static int moe_route_launch(const void* x, int ldx, int x_is_bf16, const float* router,
+                            const float* bias, int T, int D, int E, int top, bool squashed,
+                            moe_squashed_choice sq, int* idx, float* wts, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (top < 1 || top > MOE_MAX_TOP || top > E || E > 4096) return (int)hipErrorInvalidValue;
+  if (squashed && (sq.groups < 1 || sq.keep < 1 || sq.keep > sq.groups || E % sq.groups ||
+                   top > E / sq.groups * sq.keep))
+    return (int)hipErrorInvalidValue;
+  const size_t lds = ((size_t)E + MOE_ROUTE_GROUP * (MOE_THREADS / WAVE) +
+                      (squashed ? E + sq.groups : 0)) * sizeof(float);
+  const bool vec = D % 4 == 0 && (uintptr_t)router % 16 == 0;
+#define MOE_ROUTE_LAUNCH(TT, V)                                                                 \
+  if (squashed) MOE_ROUTE_LAUNCH_AS(TT, V, true); else MOE_ROUTE_LAUNCH_AS(TT, V, false)
+#define MOE_ROUTE_LAUNCH_AS(TT, V, SQ)                                                          \
+  hipLaunchKernelGGL((moe_route_kernel<TT, V, SQ>), dim3(T), dim3(MOE_THREADS), lds, stream,      \
+                     (const TT*)x, ldx, router, bias, T, D, E, top, sq, idx, wts)
+  if (x_is_bf16) {
+    if (vec) { MOE_ROUTE_LAUNCH(bf16_t, 4); } else { MOE_ROUTE_LAUNCH(bf16_t, 1); }
+  } else {
+    if (vec) { MOE_ROUTE_LAUNCH(float, 4); } else { MOE_ROUTE_LAUNCH(float, 1); }
+  }
+#undef MOE_ROUTE_LAUNCH_AS
+#undef MOE_ROUTE_LAUNCH
+  KAPPAI_RETURN_LAUNCH_STATUS();
+}
+
 extern "C" int kappai_moe_route(const void* x, int ldx, int x_is_bf16, const float* router,
                                 const float* bias, int T, int D, int E, int top, int* idx,
                                 float* wts, hipStream_t stream) {
-  if (T <= 0) return 0;
-  if (top < 1 || top > MOE_MAX_TOP || top > E || E > 4096) return (int)hipErrorInvalidValue;
-  const size_t lds = (size_t)(E + MOE_ROUTE_GROUP * (MOE_THREADS / WAVE)) * sizeof(float);
-  const bool vec = D % 4 == 0 && (uintptr_t)router % 16 == 0;
-#define MOE_ROUTE_LAUNCH(TT, V)                                                                 \
-  hipLaunchKernelGGL((moe_route_kernel<TT, V>), dim3(T), dim3(MOE_THREADS), lds, stream,          \
-                     (const TT*)x, ldx, router, bias, T, D, E, top, idx, wts)
-  if (x_is_bf16) {
-    if (vec) MOE_ROUTE_LAUNCH(bf16_t, 4); else MOE_ROUTE_LAUNCH(bf16_t, 1);
-  } else {
-    if (vec) MOE_ROUTE_LAUNCH(float, 4); else MOE_ROUTE_LAUNCH(float, 1);
-  }
-#undef MOE_ROUTE_LAUNCH
-  KAPPAI_RETURN_LAUNCH_STATUS();
+  return moe_route_launch(x, ldx, x_is_bf16, router, bias, T, D, E, top, false,
+                          moe_squashed_choice{nullptr, 1, 1, 1.0f}, idx, wts, stream);
+}
+
+extern "C" int kappai_moe_route_squashed(const void* x, int ldx, int x_is_bf16,
+                                         const float* router, const float* bias,
+                                         const float* correction, int groups, int keep,
+                                         float scale, int T, int D, int E, int top, int* idx,
+                                         float* wts, hipStream_t stream) {
+  return moe_route_launch(x, ldx, x_is_bf16, router, bias, T, D, E, top, true,
+                          moe_squashed_choice{correction, groups, keep, scale}, idx, wts, stream);
 }
 
 // The pairs sorted by expert, stably and without atomics.  The waves of one block each take a

@@ -4,6 +4,8 @@
 //   dist_bias   [heads, dist_cols] float32, added after the cap: column min(i - j, dist_cols - 1)
 //               for query position i and key position j; null: nothing
 //   sink        [heads] float32: exp(sink[h]) joins the denominator once; null: nothing
+//   keep_first  the first keep_first positions of a sequence are seen by every later one, whatever
+//               the window or chunk; 0: nothing is kept
 #pragma once
 #include <hip/hip_runtime.h>
 
@@ -22,15 +24,30 @@ struct kappai_score_mods {
   const float* dist_bias;
   int dist_cols;
   const float* sink;
+  int keep_first;
 };
 
-__host__ __device__ __forceinline__ bool kappai_mods_on(const kappai_score_mods* m) {
-  return m != nullptr && (m->softcap > 0.f || m->dist_bias != nullptr || m->sink != nullptr);
+// With kept first positions a row's keys are two runs: [0, keep) and [lo, pos], lo from
+// kappai_first_key.  The matrix-core kernels walk tiles of 32 keys; the tiles of the first run that
+// lie before the window's first tile (lo32 = lo rounded down to 32) are put right in front of it:
+// tile address kb >= lo32 holds the keys from kb on, the `kept` places before lo32 hold the keys
+// from 0 on.  With nothing kept (or a window that still reaches the beginning) kept is 0.
+__device__ __forceinline__ int kappai_kept_places(int keep, int lo32) {
+  return (min(keep, lo32) + 31) / 32 * 32;
+}
+__device__ __forceinline__ int kappai_key_at(int place, int lo32, int kept) {
+  return place >= lo32 ? place : place - (lo32 - kept);
 }
 
-// (a cap or a bias: the scores themselves change; a sink alone leaves them as they are)
+__host__ __device__ __forceinline__ bool kappai_mods_on(const kappai_score_mods* m) {
+  return m != nullptr && (m->softcap > 0.f || m->dist_bias != nullptr || m->sink != nullptr ||
+                          m->keep_first > 0);
+}
+
+// (a cap, a bias or kept positions: the scores themselves change or a row's keys are two runs; a
+// sink alone leaves them as they are)
 __host__ __device__ __forceinline__ bool kappai_mods_change_scores(const kappai_score_mods* m) {
-  return m != nullptr && (m->softcap > 0.f || m->dist_bias != nullptr);
+  return m != nullptr && (m->softcap > 0.f || m->dist_bias != nullptr || m->keep_first > 0);
 }
 
 // cap * tanh(s / cap) for the kernels that work in bfloat16: tanh(x) = 1 - 2 / (1 + e^(2x)) by the

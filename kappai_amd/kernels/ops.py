@@ -71,9 +71,9 @@ def _is_bf16(dtype) -> int:
 
 
 # ---------------------------------------------------------------------------------------
-def embed_rows(ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
+def embed_rows(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
     """float32 [T, D] rows of ``table`` ([V, D], float32 or bfloat16, or ``InFragments``: a tied
-    output head's matrix) at ``ids`` (int32)."""
+    output head's matrix) at ``ids`` (int32), times ``scale``."""
     _gpu("ids", ids, I32)
     kind = 2 if isinstance(table, InFragments) else None
     if kind is None:
@@ -82,8 +82,8 @@ def embed_rows(ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
     _need(ids.dim() == 1 and table.dim() == 2, "embed_rows: ids [T], table [V, D]")
     T, D = ids.shape[0], table.shape[1]
     out = torch.empty((T, D), dtype=F32, device=table.device)
-    check(library("elementwise").kappai_embed_rows(
-        _ptr(ids), _ptr(table), _c_int(kind), _ptr(out), _c_int(T), _c_int(D),
+    check(library("elementwise").kappai_embed_rows_scaled(
+        _ptr(ids), _ptr(table), _c_int(kind), _ptr(out), _c_int(T), _c_int(D), _c_float(scale),
         _stream()), "embed_rows")
     return out
 
@@ -821,7 +821,8 @@ def qk_norm_rope_store(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_di
 
 class ScoreModsC(ctypes.Structure):
     """``kappai_score_mods`` of csrc/score_mods.h."""
-    _fields_ = [("softcap", _c_float), ("dist_bias", _vp), ("dist_cols", _c_int), ("sink", _vp)]
+    _fields_ = [("softcap", _c_float), ("dist_bias", _vp), ("dist_cols", _c_int), ("sink", _vp),
+                ("keep_first", _c_int)]
 
 
 @dataclass(frozen=True)
@@ -830,13 +831,16 @@ class ScoreMods:
     ``softcap`` (0: nothing; else ``softcap * tanh(score / softcap)``); ``distance_bias`` float32
     [H, n], added after the cap, column ``min(i - j, n - 1)`` for query position i and key
     position j; ``sink`` float32 [H]: ``exp(sink[h])`` joins the softmax's denominator once, with
-    no key and no value behind it."""
+    no key and no value behind it; ``keep_first``: the first that many positions of a sequence are
+    seen by every later one, whatever the window or chunk, at their true distance."""
     softcap: float = 0.0
     distance_bias: Optional[torch.Tensor] = None
     sink: Optional[torch.Tensor] = None
+    keep_first: int = 0
 
     def active(self) -> bool:
-        return self.softcap > 0.0 or self.distance_bias is not None or self.sink is not None
+        return (self.softcap > 0.0 or self.distance_bias is not None or self.sink is not None
+                or self.keep_first > 0)
 
     def c_struct(self, n_heads: int) -> "ScoreModsC":
         cols = 0
@@ -849,9 +853,10 @@ class ScoreMods:
         if self.sink is not None:
             _gpu("sink", self.sink, F32)
             _need(self.sink.shape == (n_heads,), lambda: f"sink {tuple(self.sink.shape)}")
+        _need(self.keep_first >= 0, lambda: f"keep_first {self.keep_first}")
         return ScoreModsC(float(self.softcap),
                           0 if self.distance_bias is None else self.distance_bias.data_ptr(), cols,
-                          0 if self.sink is None else self.sink.data_ptr())
+                          0 if self.sink is None else self.sink.data_ptr(), int(self.keep_first))
 
 
 @dataclass
@@ -869,18 +874,22 @@ class QkPrologue:
     store_kv: bool = True
 
 
-def keys_bound(max_position: int, window: int) -> int:
+def keys_bound(max_position: int, window: int, keep_first: int = 0) -> int:
     """An upper bound of the keys a row at ``max_position`` or before sees (``window``: 0 all,
-    n > 0 a sliding window of n, n < 0 chunks of -n positions; rounded as the kernels' tiles)."""
-    return min(max_position + 1, abs(window)) + 32 if window else max_position + 1
+    n > 0 a sliding window of n, n < 0 chunks of -n positions, beside them the first
+    ``keep_first``; rounded as the kernels' tiles)."""
+    if not window:
+        return max_position + 1
+    kept = (min(keep_first, max_position + 1) + 31) // 32 * 32
+    return min(max_position + 1, abs(window)) + 32 + kept
 
 
 def decode_form(n_heads: int, n_kv_heads: int, head_dim: int, max_position: int,
-                window: int = 0) -> str:
+                window: int = 0, keep_first: int = 0) -> str:
     """Which of the two decode kernels a step takes: with few keys ("decode-block") a block per
     (row, kv head) splits them over its waves and merges in LDS; else ("decode-split") the keys
     are split over blocks, whose partial results a second kernel merges."""
-    n_keys = keys_bound(max_position, window)
+    n_keys = keys_bound(max_position, window, keep_first)
     lib = library("attention_mfma", HEAD_DIM=head_dim)
     block_waves = lib.kappai_attn_decode_block_waves(n_heads // n_kv_heads)
     return "decode-block" if block_waves and n_keys <= DECODE_BLOCK_MAX_KEYS else "decode-split"
@@ -926,7 +935,8 @@ def paged_attention(q: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: in
     leaves out, the single decoded tokens of a step that also holds prompt portions.  They go
     through the decode kernel that splits keys over blocks.
 
-    ``mods`` (``ScoreMods``): a cap on the scores, a bias by distance, a sink."""
+    ``mods`` (``ScoreMods``): a cap on the scores, a bias by distance, a sink, first positions that
+    every row sees."""
     H, G, d = n_heads, n_kv_heads, head_dim
     _need(not (window and chunk) and (window or 0) >= 0 and chunk >= 0,
           "paged_attention: a sliding window or chunks, not both")
@@ -939,6 +949,7 @@ def paged_attention(q: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: in
         mods = None
     mods_c = mods.c_struct(H) if mods is not None else None
     mods_ref = ctypes.byref(mods_c) if mods_c is not None else None
+    keep = mods.keep_first if mods is not None else 0
     _gpu("q", q, (F32, BF16), contiguous=False)
     T = q.shape[0]
     _need(q.dim() == 2 and q.shape[1] >= H * d and (q.stride(1) == 1),
@@ -994,7 +1005,7 @@ def paged_attention(q: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: in
                   "query heads a kv head) and their largest position")
             _decode_split(lib, q, H, G, d, k_pool, v_pool, row_pos, row_seg, block_tables,
                           page_size, scale, window, max_lone_position, out, lone_rows,
-                          mods_ref=mods_ref)
+                          mods_ref=mods_ref, keep_first=keep)
         return out
     _need(kernel in ("decode", "decode-block", "decode-split"),
           lambda: f"unknown attention kernel {kernel!r}")
@@ -1022,10 +1033,10 @@ def paged_attention(q: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: in
                           f"{max_position} of heads of {d}")
         qk_args = (_ptr(qk.q_norm_w), _ptr(qk.k_norm_w), _c_float(qk.eps), _ptr(qk.cos),
                    _ptr(qk.sin), _c_int(1 if qk.store_kv else 0))
-    n_keys = keys_bound(max_position, window)
     block_waves = lib.kappai_attn_decode_block_waves(H // G)
     if kernel == "decode":
-        kernel = "decode-split" if qk is not None else decode_form(H, G, d, max_position, window)
+        kernel = ("decode-split" if qk is not None
+                  else decode_form(H, G, d, max_position, window, keep))
     if kernel == "decode-block":
         _need(block_waves > 0, "too many query heads a kv head for the block form")
         _need(qk is None, "the decode kernel that keeps a row's keys in one block takes q ready "
@@ -1037,7 +1048,7 @@ def paged_attention(q: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: in
             _c_float(scale), _c_int(block_waves), mods_ref, _stream()), "attn_decode_block")
         return out
     _decode_split(lib, q, H, G, d, k_pool, v_pool, row_pos, row_seg, block_tables, page_size, scale,
-                  window, max_position, out, None, qk_args, mods_ref=mods_ref)
+                  window, max_position, out, None, qk_args, mods_ref=mods_ref, keep_first=keep)
     return out
 
 
@@ -1052,11 +1063,11 @@ def decode_splits(keys_per_wave: int, rows: int, n_kv_heads: int, n_keys: int):
 
 
 def _decode_split(lib, q, H, G, d, k_pool, v_pool, row_pos, row_seg, block_tables, page_size, scale,
-                  window, max_position, out, row_ids, qk_args=(), mods_ref=None):
+                  window, max_position, out, row_ids, qk_args=(), mods_ref=None, keep_first=0):
     """The decode kernel that splits a row's keys over blocks, and its merge, for all rows or
     (``row_ids``) some of them."""
     T = q.shape[0] if row_ids is None else row_ids.shape[0]
-    n_keys = keys_bound(max_position, window)
+    n_keys = keys_bound(max_position, window, keep_first)
     # one wave keeps the loads of `kpw` keys in flight; splits are whole numbers of that, and
     # at most DECODE_MAX_SPLITS of them are merged
     kpw = lib.kappai_attn_keys_per_wave()
@@ -1597,6 +1608,37 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, top: int,
     return idx, wts
 
 
+def moe_route_squashed(x: torch.Tensor, router: torch.Tensor, top: int, scale: float = 1.0,
+                       correction: Optional[torch.Tensor] = None, groups: int = 1,
+                       keep_groups: int = 1, bias: Optional[torch.Tensor] = None):
+    """Router logits ``z = x router^T (+ bias)`` in float32, every logit squashed by itself: score
+    ``s = sigmoid(z)``.  Chosen are the ``top`` experts with the largest ``s + correction``
+    (correction [E] float32 or None; the lowest index wins a tie) among the ``keep_groups`` best of
+    ``groups`` equal groups of neighbouring experts, a group's worth being the sum of its two
+    largest such values.  The weights are ``s * scale`` of the chosen ones.  Returns (experts [T,
+    top] int32, weights [T, top] float32), in the order of the choice."""
+    _gpu("x", x, (F32, BF16), contiguous=False)
+    _gpu("router", router, F32)
+    T, D = x.shape
+    E = router.shape[0]
+    for name, t in (("bias", bias), ("correction", correction)):
+        if t is not None:
+            _gpu(name, t, F32)
+            _need(t.shape == (E,), lambda: f"moe_route_squashed: {name} {tuple(t.shape)}")
+    _need(router.shape == (E, D) and x.stride(1) == 1 and 1 <= top <= MOE_MAX_TOP,
+          lambda: f"moe_route_squashed: x {tuple(x.shape)}, router {tuple(router.shape)}, top {top}")
+    _need(groups >= 1 and E % groups == 0 and 1 <= keep_groups <= groups
+          and top <= E // groups * keep_groups,
+          lambda: f"moe_route_squashed: {top} of {E} experts, {keep_groups} of {groups} groups")
+    idx = torch.empty((T, top), dtype=I32, device=x.device)
+    wts = torch.empty((T, top), dtype=F32, device=x.device)
+    check(library("moe").kappai_moe_route_squashed(
+        _ptr(x), _c_int(x.stride(0)), _c_int(_is_bf16(x.dtype)), _ptr(router), _ptr(bias),
+        _ptr(correction), _c_int(groups), _c_int(keep_groups), _c_float(scale), _c_int(T),
+        _c_int(D), _c_int(E), _c_int(top), _ptr(idx), _ptr(wts), _stream()), "moe_route_squashed")
+    return idx, wts
+
+
 @dataclass
 class MoePlan:
     """The step's (row, choice) pairs in expert order: ``slot_of_pair`` [T top], ``pair_of_slot``
@@ -1780,6 +1822,80 @@ def moe_combine(y: torch.Tensor, weights: torch.Tensor, plan: MoePlan,
     return out
 
 
+@dataclass
+class ExpertTerms:
+    """What a mixture's chosen experts left, not summed yet: ``y`` float32 [slots, D] in the plan's
+    order and ``weights`` [T, top].  The pass that reads it sums in the order of the choice
+    (``tanh_norm_step``), or ``combined()`` does."""
+    y: torch.Tensor
+    weights: torch.Tensor
+    plan: MoePlan
+
+    def combined(self) -> torch.Tensor:
+        return moe_combine(self.y, self.weights, self.plan)
+
+
+# ---------------------------------------------------------------------------------------
+# pointwise norms that saturate, on both sides of a sublayer
+# ---------------------------------------------------------------------------------------
+@dataclass
+class TanhNormWeights:
+    """``n(x) = tanh(alpha x) * weight + bias``, weight and bias [D] float32, one alpha a row."""
+    alpha: float
+    weight: torch.Tensor
+    bias: torch.Tensor
+
+
+def tanh_norm_step(resid: torch.Tensor, y=None, post: Optional[TanhNormWeights] = None,
+                   pre: Optional[TanhNormWeights] = None, rows: Optional[torch.Tensor] = None,
+                   rows_dtype=None) -> Optional[torch.Tensor]:
+    """One pass over the stream ``resid`` [T, D] float32: ``resid += post(y)`` in place, and the
+    rows ``pre(resid)`` in ``rows_dtype`` are returned.  ``y``: [T, D] in float32 or bfloat16,
+    float32 partial sums [S, T, D] (added in order first), ``ExpertTerms`` (summed first), or None;
+    ``post`` None: ``y`` is added as it is; ``pre`` None: no rows.  ``rows`` (int32): only these
+    rows are made, and the stream keeps its values."""
+    _gpu("resid", resid, F32)
+    _need(resid.dim() == 2, lambda: f"tanh_norm_step: resid {tuple(resid.shape)}")
+    T, D = resid.shape
+    for name, n in (("post", post), ("pre", pre)):
+        if n is not None:
+            _gpu(name + " weight", n.weight, F32)
+            _gpu(name + " bias", n.bias, F32)
+            _need(n.weight.shape == (D,) and n.bias.shape == (D,),
+                  lambda: f"tanh_norm_step: {name} {tuple(n.weight.shape)}, {tuple(n.bias.shape)}")
+    slots = wts = None
+    parts, top, isb = 1, 0, 0
+    if isinstance(y, ExpertTerms):
+        slots, wts, top, y = y.plan.slot_of_pair, y.weights, y.plan.top, y.y
+        _gpu("y", y, F32)
+        _gpu("weights", wts, F32)
+        _need(y.dim() == 2 and y.shape[1] == D and wts.shape == (T, top)
+              and slots.shape[0] == T * top, "tanh_norm_step: experts of another step")
+    elif y is not None:
+        _gpu("y", y, (F32, BF16))
+        isb = _is_bf16(y.dtype)
+        if y.dim() == 3:
+            _need(not isb, "tanh_norm_step: partial sums are float32")
+            parts = y.shape[0]
+        _need(tuple(y.shape[-2:]) == (T, D) and y.dim() in (2, 3),
+              lambda: f"tanh_norm_step: y {tuple(y.shape)} into {tuple(resid.shape)}")
+    n = T
+    if rows is not None:
+        _gpu("rows", rows, I32)
+        n = rows.shape[0]
+    out = None
+    if pre is not None:
+        out = torch.empty((n, D), dtype=rows_dtype, device=resid.device)
+    check(library("elementwise").kappai_tanh_norm_step(
+        _ptr(resid), _ptr(y), _c_int(isb), _c_int(parts), _ptr(slots), _ptr(wts), _c_int(top),
+        _c_float(post.alpha if post else 0.0), _ptr(post.weight if post else None),
+        _ptr(post.bias if post else None), _c_float(pre.alpha if pre else 0.0),
+        _ptr(pre.weight if pre else None), _ptr(pre.bias if pre else None), _ptr(rows), _c_int(n),
+        _c_int(T), _c_int(D), _ptr(out), _c_int(_is_bf16(rows_dtype) if pre else 0), _stream()),
+        "tanh_norm_step")
+    return out
+
+
 # ---------------------------------------------------------------------------------------
 # a norm on a sublayer's output, added into the residual stream
 # ---------------------------------------------------------------------------------------
@@ -1956,20 +2072,23 @@ def head_norm_rotate_store(proj: torch.Tensor, n_heads: int, n_kv_heads: int, di
                            cos: Optional[torch.Tensor], sin: Optional[torch.Tensor],
                            rot_dims: int, rot_mode: int, k_pool: torch.Tensor,
                            v_pool: torch.Tensor, row_pos: torch.Tensor, row_seg: torch.Tensor,
-                           block_tables: torch.Tensor, page_size: int) -> torch.Tensor:
+                           block_tables: torch.Tensor, page_size: int,
+                           values_are_keys: bool = False) -> torch.Tensor:
     """From ``proj`` [T, H dim + G dim + G vdim (+ more)]: every q and k head divided by the root
     mean square of its own ``dim`` places and multiplied by a weight [dim] that the heads share
     (None: no norm), then the first ``rot_dims`` places turned by the row's position (tables and
     ``rot_mode`` as ``rotate_widen_store``).  Returns queries [T, H head_size] (zeros behind
-    ``dim``); keys and values go to pools made for G kv heads of ``head_size``."""
+    ``dim``); keys and values go to pools made for G kv heads of ``head_size``.
+    ``values_are_keys``: there are no value columns; a kv head's value is its key as projected,
+    before norm and rotation."""
     H, G, d, dv, D = n_heads, n_kv_heads, dim, vdim, head_size
     _gpu("proj", proj, (F32, BF16), contiguous=False)
     T = proj.shape[0]
-    need = H * d + G * d + G * dv
+    need = H * d + G * d + (0 if values_are_keys else G * dv)
     _need(proj.dim() == 2 and proj.shape[1] >= need and proj.stride(1) == 1,
           lambda: f"head_norm_rotate_store: proj {tuple(proj.shape)} holds fewer than {need} "
                   "columns")
-    _need(H % G == 0 and d <= D and dv <= D,
+    _need(H % G == 0 and d <= D and dv <= D and (not values_are_keys or dv == d),
           lambda: f"head_norm_rotate_store: {H} heads over {G}, sizes {d} and {dv} in heads of {D}")
     for name, w in (("q_norm_w", q_norm_w), ("k_norm_w", k_norm_w)):
         if w is not None:
@@ -1997,7 +2116,8 @@ def head_norm_rotate_store(proj: torch.Tensor, n_heads: int, n_kv_heads: int, di
         _ptr(cos), _ptr(sin), _c_int(rot_dims), _c_int(rot_mode), _ptr(k_pool), _ptr(v_pool),
         _ptr(row_pos), _ptr(row_seg), _ptr(block_tables), _c_int(block_tables.shape[1]),
         _c_int(T), _c_int(H), _c_int(G), _c_int(d), _c_int(dv), _c_int(D), _c_int(page_size),
-        _ptr(q), _c_int(_is_bf16(proj.dtype)), _stream()), "head_norm_rotate_store")
+        _c_int(1 if values_are_keys else 0), _ptr(q), _c_int(_is_bf16(proj.dtype)), _stream()),
+        "head_norm_rotate_store")
     return q
 
 

@@ -152,8 +152,8 @@ class Model:
         calls = []
         if self.embedding_norm is not None:
             return None            # the walk from C knows no norm between embedding and layers
-        if getattr(self.head, "softcap", 0.0):
-            return None            # nor a cap on the logits
+        if getattr(self.head, "softcap", 0.0) or getattr(self.embedding, "scale", 1.0) != 1.0:
+            return None            # nor a cap on the logits or a factor on the embedded rows
         if any(call.enters is not None for call in self.schedule):
             return None            # nor parts that work on the stream between two blocks
         for ci, call in enumerate(self.schedule):
@@ -207,7 +207,7 @@ class Model:
                 h = block.forward(h, batch, view, shared_cache=shared)
         if batch.n_logit_rows == 0:
             return torch.empty((0, self.vocab_size), dtype=torch.float32, device=x.device)
-        delta = summed_delta(self.final_norm, h.delta)
+        delta = summed_delta(self.final_norm, h.delta, h.resid)
         if (getattr(self.final_norm, "can_defer", False)
                 and getattr(self.head, "takes_deferred_rows", False)):
             made = (isinstance(delta, ops.ScaledRows)

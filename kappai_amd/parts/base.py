@@ -93,11 +93,16 @@ class Norm(Part):
         raise NotImplementedError
 
 
-def summed_delta(norm: Norm, delta):
+def summed_delta(norm: Norm, delta, resid: Optional[torch.Tensor] = None):
     """``delta`` as ``norm`` takes it: partial sums [S, T, width] are added up first unless the
     norm adds them itself, and what a product returns that has added its result into the
-    residual itself (``ops.Added``) becomes None unless the norm knows of such things."""
+    residual itself (``ops.Added``) becomes None unless the norm knows of such things.  A
+    ``NormedUpdate`` is applied to ``resid`` here unless the norm does that in its own pass
+    (``takes_normed_update``)."""
     from ..kernels import ops
+    if isinstance(delta, NormedUpdate) and not getattr(norm, "takes_normed_update", False):
+        delta.norm.norm_output(resid, delta.y)
+        return None
     if isinstance(delta, ops.Added) and not getattr(norm, "can_defer", False):
         return None                  # a product has added its result into the residual itself
     if (isinstance(delta, torch.Tensor) and delta.dim() == 3
@@ -175,6 +180,17 @@ class WeightedTerms:
     scale_a: float
     b: torch.Tensor
     scale_b: float
+
+
+@dataclass
+class NormedUpdate:
+    """A sublayer's result that passes a norm of its own on the way into the stream, not applied
+    yet: ``resid += norm(y)``.  ``y``: [T, width], float32 partial sums [S, T, width], or what a
+    mixture's experts left (``ops.ExpertTerms``, for a norm with ``takes_expert_terms``).  The pass
+    that reads the stream next applies it (a norm with ``takes_normed_update``), or
+    ``norm.norm_output`` does."""
+    y: object
+    norm: "Norm"
 
 
 @dataclass

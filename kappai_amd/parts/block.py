@@ -9,8 +9,8 @@ from ..kernels import ops
 from ..weights.spec import TensorSpec
 from ctypes import Structure
 
-from .base import (Block, FeedForward, Hidden, Mixer, Norm, StreamUpdate, register_part,
-                   summed_delta)
+from .base import (Block, FeedForward, Hidden, Mixer, Norm, NormedUpdate, StreamUpdate,
+                   register_part, summed_delta)
 from ..weights.spec import INIT_CONNECT, VECTOR
 from .cdesc import NormPartDesc, PartDesc, defined_together
 
@@ -105,7 +105,7 @@ class PreNormBlock(Block):
 
     @staticmethod
     def _normed(norm, resid, delta, consumer):
-        delta = summed_delta(norm, delta)
+        delta = summed_delta(norm, delta, resid)
         if getattr(consumer, "takes_deferred_rows", False) and _takes_defer(norm):
             return norm.add_norm(resid, delta, defer=True)
         return norm.add_norm(resid, delta)
@@ -190,7 +190,7 @@ class ConvInputBlock(Block):
 
     @staticmethod
     def _read(norm, conv, resid, delta, batch, state):
-        delta = summed_delta(norm, delta)
+        delta = summed_delta(norm, delta, resid)
         if conv is None:
             return norm.add_norm(resid, delta)
         if batch.max_segment_rows == 1 and hasattr(norm, "add_norm_conv_step"):
@@ -400,3 +400,75 @@ class HyperConnectionBlock(Block):
 
 
 register_part("block", "hyper_connection", HyperConnectionBlock)
+
+
+class SandwichNormBlock(Block):
+    """``x += out1(mixer(norm1(x))); x += out2(feed_forward(norm2(x)))``: a norm before and a norm
+    behind every sublayer.  ``feed_forward`` (with its two norms) may be None.
+
+    What a sublayer returns is not normed when it is made: it travels as a ``NormedUpdate`` to the
+    norm that reads the stream next.  Where that norm applies such updates itself
+    (``takes_normed_update``), a sublayer costs one pass over the stream: norm of the update, sum,
+    norm of the new stream.  The norms behind the sublayers must know ``norm_output``."""
+
+    def __init__(self, mixer_norm: Norm, mixer: Mixer, mixer_out_norm: Norm,
+                 ffn_norm: Norm = None, feed_forward: FeedForward = None,
+                 ffn_out_norm: Norm = None):
+        if len({p is None for p in (ffn_norm, feed_forward, ffn_out_norm)}) != 1:
+            raise ValueError("a feed-forward and its two norms come together")
+        for n in (mixer_out_norm, ffn_out_norm):
+            if n is not None and not hasattr(n, "norm_output"):
+                raise ValueError(f"{type(n).__name__} cannot norm a sublayer's output into the "
+                                 "stream (no norm_output)")
+        self.mixer_norm, self.mixer, self.mixer_out_norm = mixer_norm, mixer, mixer_out_norm
+        self.ffn_norm, self.feed_forward = ffn_norm, feed_forward
+        self.ffn_out_norm = ffn_out_norm
+
+    def _parts(self):
+        return tuple(p for p in (self.mixer_norm, self.mixer, self.mixer_out_norm, self.ffn_norm,
+                                 self.feed_forward, self.ffn_out_norm) if p is not None)
+
+    @property
+    def capturable(self) -> bool:
+        return all(p.capturable for p in self._parts())
+
+    @property
+    def step_tables(self):
+        out = []
+        for p in self._parts():
+            asked = p.step_tables
+            if asked is not None:
+                out += list(asked) if isinstance(asked, (list, tuple)) else [asked]
+        return out
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return [s for p in self._parts() for s in p.tensor_specs()]
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        for p in self._parts():
+            p.bind(tensors)
+
+    @staticmethod
+    def _read(norm, resid, delta):
+        return norm.add_norm(resid, summed_delta(norm, delta, resid))
+
+    def forward(self, h: Hidden, batch, cache, shared_cache: bool = False) -> Hidden:
+        resid = h.resid
+        x = self._read(self.mixer_norm, resid, h.delta)
+        mixed = self.mixer.forward(x, batch, cache, shared_cache=shared_cache)
+        update = NormedUpdate(mixed, self.mixer_out_norm)
+        if self.feed_forward is None:
+            return Hidden(resid, update)
+        x = self._read(self.ffn_norm, resid, update)
+        if (getattr(self.feed_forward, "hands_on_terms", False)
+                and getattr(self.ffn_out_norm, "takes_expert_terms", False)):
+            out = self.feed_forward.forward(x, batch, terms=True)
+        else:
+            out = self.feed_forward.forward(x, batch)
+        return Hidden(resid, NormedUpdate(out, self.ffn_out_norm))
+
+    def weight_bytes(self) -> int:
+        return sum(p.weight_bytes() for p in self._parts())
+
+
+register_part("block", "sandwich_norm", SandwichNormBlock)

@@ -12,12 +12,15 @@ from .linear import Linear
 
 
 class TokenEmbedding(Part):
-    """Rows of the table widened to float32, without a scale
-    (kappai: src/recipe/scratch.c:195-235)."""
+    """Rows of the table widened to float32, times a constant
+    (kappai, without one: src/recipe/scratch.c:195-235)."""
 
-    def __init__(self, name: str, vocab: int, width: int, suffix: str = ".weight"):
-        """``suffix``: how the table's tensor name ends in the checkpoint."""
+    def __init__(self, name: str, vocab: int, width: int, suffix: str = ".weight",
+                 scale: float = 1.0):
+        """``suffix``: how the table's tensor name ends in the checkpoint.  ``scale``: a factor on
+        the embedded rows (a tied output head reads the table without it)."""
         self.name, self.vocab, self.width = name, vocab, width
+        self.scale = float(scale)
         self.tensor_name = name + suffix
         self.table: Optional[torch.Tensor] = None
 
@@ -29,6 +32,8 @@ class TokenEmbedding(Part):
 
     def forward(self, tokens: torch.Tensor) -> torch.Tensor:
         with profile.scope("embd"):
+            if self.scale != 1.0:
+                return ops.embed_rows(tokens, self.table, scale=self.scale)
             return ops.embed_rows(tokens, self.table)
 
     def c_table(self):

@@ -3,7 +3,11 @@
 weights are the softmax over the chosen logits alone; the output is the weighted sum of the
 chosen experts' ``W_down (silu(W_gate h) * W_up h)``.  Experts have no biases.  ``activation``
 "relu_squared": the experts have no gate, ``W_down relu(W_up h)^2``.  ``router_bias``: a bias [E]
-on the router's logits.  ``shared_hidden``: one more expert of that size and the same form
+on the router's logits.  ``scoring`` "sigmoid": the router squashes every logit by itself, ``s =
+sigmoid(z)``; the choice goes by ``s`` plus a learned ``correction`` [E] (where there is one), among
+the experts of the ``keep_groups`` best of ``groups`` equal groups of neighbours (a group's worth:
+the sum of its two largest such values), and the weights are the chosen experts' ``s`` times
+``weight_scale``, without the correction and not renormalised.  ``shared_hidden``: one more expert of that size and the same form
 (``<prefix>shared.``) runs for every row, and its result is added with weight one.
 
 The step's (row, choice) pairs are sorted by expert on the GPU and the experts' products run
@@ -22,13 +26,27 @@ from .linear import Linear
 
 
 class MixtureOfExperts(FeedForward):
+    SCORINGS = ("softmax", "sigmoid")
+
     def __init__(self, prefix: str, width: int, hidden: int, experts: int, top: int,
                  dtype: torch.dtype, names=None, weight_suffix: str = ".weight",
                  activation: str = "silu_gated", router_bias: bool = False,
-                 shared_hidden: Optional[int] = None, bias_suffix: str = ".bias"):
+                 shared_hidden: Optional[int] = None, bias_suffix: str = ".bias",
+                 scoring: str = "softmax", correction: bool = False, groups: int = 1,
+                 keep_groups: int = 1, weight_scale: float = 1.0):
         n = {"router": "router", "expert": "e{}.", "gate": "gate", "up": "up", "down": "down",
-             "shared": "shared."}
+             "shared": "shared.", "correction": "correction"}
         n.update(names or {})
+        if scoring not in self.SCORINGS:
+            raise ValueError(f"{prefix}: unknown router scoring {scoring!r}; known: "
+                             f"{', '.join(self.SCORINGS)}")
+        if scoring == "softmax" and (correction or groups != 1 or weight_scale != 1.0):
+            raise ValueError(f"{prefix}: a correction, groups and a weight scale go with the "
+                             "sigmoid scoring")
+        if not (groups >= 1 and experts % groups == 0 and 1 <= keep_groups <= groups
+                and top <= experts // groups * keep_groups):
+            raise ValueError(f"{prefix}: {top} experts a token from the best {keep_groups} of "
+                             f"{groups} groups of {experts} experts")
         if activation not in ("silu_gated", "relu_squared"):
             raise ValueError(f"{prefix}: unknown expert activation {activation!r}; known: "
                              "silu_gated, relu_squared")
@@ -41,6 +59,10 @@ class MixtureOfExperts(FeedForward):
         self._kinds = ("gate", "up", "down") if self.gated else ("up", "down")
         self._router = prefix + n["router"] + weight_suffix
         self._router_bias = prefix + n["router"] + bias_suffix if router_bias else None
+        self.scoring, self.weight_scale = scoring, float(weight_scale)
+        self.groups, self.keep_groups = int(groups), int(keep_groups)
+        self._correction = prefix + n["correction"] if correction else None
+        self.correction: Optional[torch.Tensor] = None
         self._expert = [{k: prefix + n["expert"].format(e) + n[k] + weight_suffix
                          for k in self._kinds} for e in range(self.E)]
         self.router_bias: Optional[torch.Tensor] = None
@@ -60,6 +82,8 @@ class MixtureOfExperts(FeedForward):
         specs = [TensorSpec(self._router, (self.E, self.width), MATRIX, INIT_NORMAL)]
         if self._router_bias:
             specs.append(TensorSpec(self._router_bias, (self.E,), VECTOR, INIT_SMALL))
+        if self._correction:
+            specs.append(TensorSpec(self._correction, (self.E,), VECTOR, INIT_SMALL))
         for names in self._expert:
             if self.gated:
                 specs.append(TensorSpec(names["gate"], (self.hidden, self.width), MATRIX,
@@ -83,6 +107,8 @@ class MixtureOfExperts(FeedForward):
             return w
         if self._router_bias:
             self.router_bias = tensors[self._router_bias].to(torch.float32).contiguous()
+        if self._correction:
+            self.correction = tensors[self._correction].to(torch.float32).contiguous()
         self.w_gate = stacked("gate") if self.gated else None
         self.w_up = stacked("up")
         self.w_down = stacked("down")
@@ -90,9 +116,22 @@ class MixtureOfExperts(FeedForward):
             self.shared_up.bind(tensors)
             self.shared_down.bind(tensors)
 
-    def forward(self, x, batch):
+    @property
+    def hands_on_terms(self) -> bool:
+        """``forward(..., terms=True)`` leaves the sum over the chosen experts to the caller
+        (``ops.ExpertTerms``)."""
+        return self.shared_up is None
+
+    def _route(self, x):
+        if self.scoring == "sigmoid":
+            return ops.moe_route_squashed(x, self.router, self.top, self.weight_scale,
+                                          correction=self.correction, groups=self.groups,
+                                          keep_groups=self.keep_groups, bias=self.router_bias)
+        return ops.moe_route(x, self.router, self.top, bias=self.router_bias)
+
+    def forward(self, x, batch, terms: bool = False):
         with profile.scope("router"):
-            chosen, weights = ops.moe_route(x, self.router, self.top, bias=self.router_bias)
+            chosen, weights = self._route(x)
             plan = ops.moe_plan(chosen, self.E)
         also = None
         if self.shared_up is not None:
@@ -105,6 +144,8 @@ class MixtureOfExperts(FeedForward):
                    else ops.moe_experts_activated(x, self.w_up, plan))
         with profile.scope("matmul_ffn_down", 0):
             y = ops.moe_experts_down(act, self.w_down, plan)
+            if terms and also is None:
+                return ops.ExpertTerms(y, weights, plan)
             return ops.moe_combine(y, weights, plan, also=also)
 
     def weight_bytes(self) -> int:

@@ -9,7 +9,7 @@ import torch
 
 from ..kernels import ops, profile, tuning
 from ..weights.spec import INIT_ONES, INIT_SMALL, VECTOR, TensorSpec
-from .base import Norm, StreamUpdate, WeightedTerms, register_part
+from .base import Norm, NormedUpdate, StreamUpdate, WeightedTerms, register_part
 from .cdesc import FoldDesc
 
 
@@ -149,3 +149,65 @@ class LayerNorm(Norm):
 
 
 register_part("norm", "layernorm", LayerNorm)
+
+
+class TanhNorm(Norm):
+    """``tanh(alpha * x) * w + b`` place by place ("dynamic tanh"): a norm that saturates instead
+    of dividing by a statistic of the row, with one learned ``alpha`` and the vectors ``w`` and
+    ``b`` [width]; in float32.  As no place looks at another, one pass does everything that stands
+    between two sublayers: the norm on what the first returned (``NormedUpdate``; the sum over a
+    mixture's experts or over a product's partial sums included), the residual sum, and the norm
+    in front of the second."""
+
+    takes_partial_sums = True      # the kernel adds [S, T, width] partial sums itself, in order
+    takes_normed_update = True     # and norms a pending update on the way into the stream
+    takes_expert_terms = True      # and sums what a mixture's chosen experts left
+
+    def __init__(self, name: str, width: int, dtype: torch.dtype, suffix: str = "",
+                 alpha_suffix: str = ".alpha", bias_suffix: str = ".b"):
+        self.name, self.width, self.dtype = name, width, dtype
+        self.tensor_name = name + suffix
+        self.alpha_name, self.bias_name = name + alpha_suffix, name + bias_suffix
+        self.weights: Optional[ops.TanhNormWeights] = None
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return [TensorSpec(self.tensor_name, (self.width,), VECTOR, INIT_ONES),
+                TensorSpec(self.alpha_name, (), VECTOR, INIT_ONES),
+                TensorSpec(self.bias_name, (self.width,), VECTOR, INIT_SMALL)]
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.weights = ops.TanhNormWeights(
+            float(tensors[self.alpha_name]),
+            tensors[self.tensor_name].to(torch.float32).contiguous(),
+            tensors[self.bias_name].to(torch.float32).contiguous())
+
+    def norm_output(self, resid, y, rows_dtype=None, add: bool = True):
+        """``resid += norm(y)`` in float32, in place; returns the new stream rounded to
+        ``rows_dtype`` (None: nothing)."""
+        if not add or isinstance(y, WeightedTerms):
+            raise ValueError("this norm adds one sublayer's result to a stream that is there")
+        with profile.scope("rmsnorm"):
+            ops.tanh_norm_step(resid, y, post=self.weights)
+            return None if rows_dtype is None else ops.cast(resid, rows_dtype)
+
+    def add_norm(self, resid, delta, rows=None):
+        """The ``Norm`` interface; ``delta`` may also be a ``NormedUpdate``, or ``ops.ExpertTerms``
+        to add as they are."""
+        post = None
+        if isinstance(delta, NormedUpdate):
+            if isinstance(delta.norm, TanhNorm):
+                delta, post = delta.y, delta.norm.weights
+            else:
+                delta.norm.norm_output(resid, delta.y)
+                delta = None
+        if isinstance(delta, ops.Added):
+            delta = None             # the sum is in ``resid`` already
+        with profile.scope("rmsnorm" if rows is None else "logits_norm"):
+            return ops.tanh_norm_step(resid, delta, post=post, pre=self.weights, rows=rows,
+                                      rows_dtype=self.dtype)
+
+    def weight_bytes(self) -> int:
+        return self.width * 8
+
+
+register_part("norm", "tanh_norm", TanhNorm)

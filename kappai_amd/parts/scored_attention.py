@@ -14,7 +14,9 @@ position instead of the norm and the temperature; ``bias``: q, k and v have bias
 ``values_from_keys``: there is no ``W_v``, a kv head's value is its key as projected, before the
 rotation.  ``head_qk_norm``: every q and k head is divided by the root mean square of its own
 ``dim`` places and multiplied by a weight of that size which all heads share, before the
-rotation.  ``sink_value``: the sink is this constant score for every head (0: a one in the
+rotation; without ``head_norm_weight`` there is no such weight.  ``keep_first``: with a window (or
+chunks) every position also sees the first ``keep_first`` positions of its sequence, at their true
+distance.  ``sink_value``: the sink is this constant score for every head (0: a one in the
 softmax's denominator) and no tensor.  ``head_gate``: a map ``W_g`` [heads, width] of the mixer's
 input gives one number a head, and the head's result is multiplied by its sigmoid before ``W_o``.
 ``bucket``: a distance below half the
@@ -73,7 +75,8 @@ class ScoredAttention(Mixer):
                  names=None, weight_suffix: str = ".weight", chunk: Optional[int] = None,
                  position=None, bias: bool = False, bias_suffix: str = ".bias",
                  values_from_keys: bool = False, head_qk_norm: bool = False,
-                 sink_value: Optional[float] = None, head_gate: bool = False):
+                 sink_value: Optional[float] = None, head_gate: bool = False,
+                 head_norm_weight: bool = True, keep_first: int = 0):
         n = {"q": "q", "k": "k", "v": "v", "o": "o", "q_norm": "q.norm", "k_norm": "k.norm",
              "rel": "rel", "sink": "sink", "gate": "g"}
         n.update(names or {})
@@ -96,10 +99,13 @@ class ScoredAttention(Mixer):
         self.position, self.values_from_keys = position, bool(values_from_keys)
         self.head_qk_norm, self.head_gate = bool(head_qk_norm), bool(head_gate)
         self.sink_value = None if sink_value is None else float(sink_value)
-        if self.head_qk_norm and (whole_qk_norm or temp_coef or self.values_from_keys):
+        self.head_norm_weight = bool(head_norm_weight)
+        self.keep_first = int(keep_first) if self.window or self.chunk else 0
+        if keep_first < 0:
+            raise ValueError(f"{prefix}: keep_first must not be negative, got {keep_first}")
+        if self.head_qk_norm and (whole_qk_norm or temp_coef):
             raise ValueError(f"{prefix}: the norm of every head by itself goes with neither the "
-                             "whole-projection norm, the query temperature nor values that are "
-                             "the keys")
+                             "whole-projection norm nor the query temperature")
         if self.sink_value is not None and sink:
             raise ValueError(f"{prefix}: a learned sink or a constant one, not both")
         if position is not None and (whole_qk_norm or temp_coef):
@@ -135,14 +141,15 @@ class ScoredAttention(Mixer):
 
     def cache_spec(self):
         # (pages of chunks that lie behind stay with the request: only a window gives them back)
-        return PagedKV(self.G, self.head_size, self.window)
+        return PagedKV(self.G, self.head_size, self.window,
+                       self.keep_first if self.window else 0)
 
     def tensor_specs(self) -> List[TensorSpec]:
         specs = self.qkv.tensor_specs() + self.out.tensor_specs()
         if self.whole_qk_norm:
             specs.append(TensorSpec(self._names["q_norm"], (self.H * self.d,), VECTOR, INIT_ONES))
             specs.append(TensorSpec(self._names["k_norm"], (self.G * self.d,), VECTOR, INIT_ONES))
-        if self.head_qk_norm:
+        if self.head_qk_norm and self.head_norm_weight:
             specs.append(TensorSpec(self._names["q_norm"], (self.d,), VECTOR, INIT_ONES))
             specs.append(TensorSpec(self._names["k_norm"], (self.d,), VECTOR, INIT_ONES))
         if self.bias_buckets:
@@ -163,7 +170,10 @@ class ScoredAttention(Mixer):
             self.out.set_weight(wide.reshape(w.shape[0], H * D).contiguous())
         else:
             self.out.bind(tensors)
-        if self.whole_qk_norm or self.head_qk_norm:
+        if self.head_qk_norm and not self.head_norm_weight:
+            self.q_norm_w = self.k_norm_w = torch.ones(
+                self.d, dtype=torch.float32, device=tensors[self._o_name].device)
+        elif self.whole_qk_norm or self.head_qk_norm:
             self.q_norm_w = tensors[self._names["q_norm"]].to(torch.float32).contiguous()
             self.k_norm_w = tensors[self._names["k_norm"]].to(torch.float32).contiguous()
         bias = sink = None
@@ -174,7 +184,7 @@ class ScoredAttention(Mixer):
         elif self.sink_value is not None:
             sink = torch.full((H,), self.sink_value, dtype=torch.float32,
                               device=tensors[self._o_name].device)
-        self.mods = ops.ScoreMods(self.softcap, bias, sink)
+        self.mods = ops.ScoreMods(self.softcap, bias, sink, self.keep_first)
 
     def forward(self, x, batch, cache, shared_cache: bool = False):
         if shared_cache:
@@ -191,7 +201,8 @@ class ScoredAttention(Mixer):
                     proj, H, G, self.d, self.dv, D, self.q_norm_w, self.k_norm_w, self.norm_eps,
                     rot.cos if rot else None, rot.sin if rot else None,
                     rot.rot_dim if rot else 0, rot.mode if rot else ops.ROT_NONE, k_pool, v_pool,
-                    batch.row_pos, batch.row_seg, tables, cache.page_size)
+                    batch.row_pos, batch.row_seg, tables, cache.page_size,
+                    values_are_keys=self.values_from_keys)
             elif self.position is not None or self.values_from_keys:
                 rot = (self.position.rotation(x.device, batch.max_position)
                        if self.position is not None else None)

@@ -12,8 +12,8 @@ F32, BF16 = torch.float32, torch.bfloat16
 ROT_NONE, ROT_HALF, ROT_INTERLEAVED = 0, 1, 2
 
 
-def embed_rows(ids, table):
-    return table[ids.long()].to(F32)
+def embed_rows(ids, table, scale=1.0):
+    return table[ids.long()].to(F32) * scale
 
 
 def add_rmsnorm(resid, delta, weight, eps, out_dtype, rows=None, write_resid=True,
@@ -170,6 +170,8 @@ def paged_attention(q, n_heads, n_kv_heads, head_dim, k_pool, v_pool, row_pos, r
             lo = p - p % chunk
         bt = block_tables[int(row_seg[t])]
         idx = torch.arange(lo, p + 1)
+        if mods is not None and mods.keep_first:
+            idx = torch.cat([torch.arange(min(mods.keep_first, lo)), idx])
         pages = bt[(idx // page_size).long()].long()
         assert bool((pages >= 0).all()), "attention reads a page that was given back"
         keys = k_pool[pages, :, (idx % page_size).long(), :].to(F32)     # [n, G, d]
@@ -688,6 +690,44 @@ def moe_route(x, router, top, bias=None):
     return chosen.to(torch.int32), torch.softmax(best, dim=-1)
 
 
+def moe_route_squashed(x, router, top, scale=1.0, correction=None, groups=1, keep_groups=1,
+                       bias=None):
+    z = x.to(F32) @ router.T
+    if bias is not None:
+        z = z + bias
+    s = torch.sigmoid(z)
+    c = s if correction is None else s + correction
+    T, E = s.shape
+    if keep_groups < groups:
+        by_group = c.reshape(T, groups, E // groups)
+        worth = by_group.topk(min(2, E // groups), dim=-1).values.sum(-1)
+        kept = torch.zeros((T, groups), dtype=torch.bool)
+        kept.scatter_(1, worth.topk(keep_groups, dim=-1).indices, True)
+        c = by_group.masked_fill(~kept[:, :, None], -float("inf")).reshape(T, E)
+    chosen = c.topk(top, dim=-1).indices
+    return chosen.to(torch.int32), s.gather(1, chosen) * scale
+
+
+def tanh_norm_step(resid, y=None, post=None, pre=None, rows=None, rows_dtype=None):
+    x = resid
+    if y is not None:
+        if hasattr(y, "combined"):
+            y = y.combined()
+        u = torch.zeros_like(resid)
+        for p in (y if y.dim() == 3 else y[None]):
+            u = u + p.to(F32)
+        if post is not None:
+            u = torch.tanh(post.alpha * u) * post.weight + post.bias
+        x = resid + u
+        if rows is None:
+            resid.copy_(x)
+    if pre is None:
+        return None
+    if rows is not None:
+        x = x[rows.long()]
+    return (torch.tanh(pre.alpha * x) * pre.weight + pre.bias).to(rows_dtype)
+
+
 def moe_plan(experts, n_experts):
     return _Plan(experts)
 
@@ -733,14 +773,14 @@ def moe_combine(y, weights, plan, also=None):
 
 def head_norm_rotate_store(proj, n_heads, n_kv_heads, dim, vdim, head_size, q_norm_w, k_norm_w,
                            eps, cos, sin, rot_dims, rot_mode, k_pool, v_pool, row_pos, row_seg,
-                           block_tables, page_size):
+                           block_tables, page_size, values_are_keys=False):
     H, G, d, dv, D = n_heads, n_kv_heads, dim, vdim, head_size
     T = proj.shape[0]
     p = proj.to(F32)
     pos = row_pos.long()
     q = p[:, :H * d].reshape(T, H, d)
     k = p[:, H * d:(H + G) * d].reshape(T, G, d)
-    v = p[:, (H + G) * d:(H + G) * d + G * dv].reshape(T, G, dv)
+    v = k if values_are_keys else p[:, (H + G) * d:(H + G) * d + G * dv].reshape(T, G, dv)
     if q_norm_w is not None:
         q = q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * q_norm_w
     if k_norm_w is not None:
@@ -800,7 +840,7 @@ def activate(x, kind=0):
     return (r * r).to(x.dtype)
 
 
-ALL = ["moe_experts_activated", "head_norm_rotate_store", "hyper_step", "rows_rmsnorm", "sigmoid_gate",
+ALL = ["moe_route_squashed", "tanh_norm_step", "moe_experts_activated", "head_norm_rotate_store", "hyper_step", "rows_rmsnorm", "sigmoid_gate",
        "softcap_rows", "activate", "add_group_rmsnorm", "add_group_rmsnorm_canon_step", "canon_conv", "scale_add_positions", "glu", "mingru_scan", "diff_store",
        "diff_combine", "moe_route", "moe_plan", "moe_experts_gated", "moe_experts_down", "moe_combine",
        "output_norm_add", "projection_norm_store", "latent_store", "headwise_linear", "conv_silu",
