@@ -117,7 +117,11 @@ COMPARISONS = {"w1024": ("dapipel-w1024", "lfm2-like-w1024"),
                # relative: the same two attention parts, scores worked on before the softmax, a
                # latent for keys and values) and beside the same LFM2 shapes
                "sibodra-w1024": ("sibodra-w1024", "dukolorn-w1024", "lfm2-like-w1024"),
-               "sibodra-w2048": ("sibodra-w2048", "dukolorn-w2048", "lfm2-like-w2048")}
+               "sibodra-w2048": ("sibodra-w2048", "dukolorn-w2048", "lfm2-like-w2048"),
+               # the Nuzivik decoder beside the Sibodra decoder of equal size (its closest
+               # relative: the same scored attention, a mixture of experts) and the LFM2 shapes
+               "nuzivik-w1024": ("nuzivik-w1024", "sibodra-w1024", "lfm2-like-w1024"),
+               "nuzivik-w2048": ("nuzivik-w2048", "sibodra-w2048", "lfm2-like-w2048")}
 
 
 def stage_table(runner, entries_of, reps):
@@ -576,13 +580,14 @@ def main() -> int:
                          "the greedy choice (1: none)")
     ap.add_argument("--compare", default="", metavar="SIZES",
                     help="instead of the headline run: prompt and decode steps of the Dapipel, "
-                         "Dukolorn, Zumuzen or Sibodra decoder beside the LFM2 shape of equal size, at these sizes (comma "
-                         "separated: " + ", ".join(sorted(COMPARISONS)) + "; 'all')")
+                         "Dukolorn, Zumuzen, Sibodra or Nuzivik decoder beside the LFM2 shape of "
+                         "equal size, at these sizes (comma separated: " + ", ".join(sorted(COMPARISONS)) + "; 'all')")
     args = ap.parse_args()
     if args.compare:
         keys = (sorted(k for k in COMPARISONS if k.startswith("w")) if args.compare == "all"
                 else sorted(k for k in COMPARISONS if k.startswith(args.compare + "-"))
-                if args.compare in ("dukolorn", "zumuzen", "sibodra") else args.compare.split(","))
+                if args.compare in ("dukolorn", "zumuzen", "sibodra", "nuzivik")
+                else args.compare.split(","))
         for k in keys:
             if k not in COMPARISONS:
                 print(f"bench.py: no comparison {k!r}; known: {', '.join(sorted(COMPARISONS))}")

@@ -243,6 +243,34 @@ SHAPES.update({
 })
 
 
+def _nuzivik(width, n_layers, heads, kv_heads, dim, window, keep_first, buckets, bias_max, ff,
+             experts, top, groups, keep_groups, vocab=65536) -> dict:
+    """``n_layers`` equal layers: windowed attention that keeps the first ``keep_first`` positions,
+    and a mixture of ``experts`` experts of ``ff // top`` in groups."""
+    layer = {"type": "attention",
+             "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
+                       "scale": dim ** -0.5, "bias_max": bias_max, "buckets": buckets,
+                       "mask": {"size": window, "keep_first": keep_first}},
+             "mlp": {"kind": "moe", "expert": {"ff": ff // top},
+                     "router": {"experts": experts, "top": top, "scale": 1.0,
+                                "groups": {"count": groups, "keep": keep_groups}}}}
+    return {"architecture": "Nuzivik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+            "embedding": {"scale": width ** 0.5},
+            "layers": [copy.deepcopy(layer) for _ in range(n_layers)]}
+
+
+SHAPES.update({
+    # eight layers at a width of 1024: 16 heads of 64 on 4 kv heads, a window of 1024 beside the
+    # first 64 positions, 32 rows of distance bias; 16 experts of 1152 in 4 groups of which 2 can
+    # be chosen from, 4 a token (4608 active)
+    "nuzivik-w1024": _nuzivik(1024, 8, 16, 4, 64, 1024, 64, 32, 1024, 4608, 16, 4, 4, 2),
+    # the same at a width of 2048: 32 heads on 8 kv heads, experts of 2048 (8192 active)
+    "nuzivik-w2048": _nuzivik(2048, 8, 32, 8, 64, 1024, 64, 32, 1024, 8192, 16, 4, 4, 2),
+    # a tiny one for smoke runs
+    "nuzivik-tiny": _nuzivik(64, 3, 4, 2, 8, 24, 3, 8, 40, 96, 6, 2, 3, 2, vocab=256),
+})
+
+
 def named_shape(name: str) -> dict:
     """A copy of the configuration called ``name`` (any case), or a ``KeyError`` naming them all."""
     key = name.strip().lower()

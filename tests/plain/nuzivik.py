@@ -133,7 +133,8 @@ def moe_ff(h, t, p: str, mlp: dict, rounding=None, margins: list = None):
         order, gap = choose(s[i], corr, router)
         gaps.append(gap)
         for e in order:
-            out[i] += s[i, e] * router["scale"] * expert(h[i:i + 1], t, f"{p}e{e}.", rounding)[0]
+            w = s[i, e] * router.get("scale", 1.0)
+            out[i] += w * expert(h[i:i + 1], t, f"{p}e{e}.", rounding)[0]
     if margins is not None:
         margins.append(torch.tensor(gaps, dtype=F64))
     return out
@@ -144,7 +145,8 @@ def forward(cfg: dict, t: Dict[str, torch.Tensor], tokens: List[int], rounding=N
     """Float64 logits [len(tokens), vocab].  ``layers_out``: gets the stream after every layer;
     ``margins``: gets every router's margins (``moe_ff``)."""
     eps = cfg["norm"]["eps"]
-    x = t["embed"].to(F64)[torch.tensor(tokens, dtype=torch.long)] * cfg["embedding"]["scale"]
+    x = t["embed"].to(F64)[torch.tensor(tokens, dtype=torch.long)]
+    x = x * (cfg.get("embedding") or {}).get("scale", 1.0)
     for i, layer in enumerate(cfg["layers"]):
         p = f"l{i}."
         if layer["type"] != "attention":
