@@ -30,6 +30,7 @@ static_assert(HEAD_DIM % 16 == 0 && HEAD_DIM >= 16 && HEAD_DIM <= 256, "unsuppor
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
+typedef __attribute__((ext_vector_type(4), aligned(4))) float f32x4_any_t;   // at any float
 typedef __attribute__((ext_vector_type(16))) float f32x16_t;
 typedef __attribute__((ext_vector_type(4))) uint32_t u32x4_t;
 typedef __attribute__((ext_vector_type(2))) uint32_t u32x2_t;
@@ -146,8 +147,12 @@ __device__ __forceinline__ u32x4_t load_k8(const bf16_t* __restrict__ k_pool,
 // first positions the tiles that hold them stand in front of the window's first tile
 // (kappai_key_at).  A sink may join the denominator with or without MODS.
 #define P_BIAS_MAX 2048
+#define P_BIAS_EDGE 64
+// waves a SIMD that the registers are held down to (2,048 rows of 32 heads of 64: 132 us with one
+// wave, which is what the compiler settles on by itself, 76 us with two)
+#define P_MIN_WAVES (HEAD_DIM <= 96 ? 2 : 1)
 template <bool MODS>
-__global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
+__global__ __launch_bounds__(P_NW * WAVE, P_MIN_WAVES) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pool,
     const bf16_t* __restrict__ vt_pool, bf16_t* __restrict__ out, int out_stride,
     const int* __restrict__ q_tiles, const int* __restrict__ row_pos,
@@ -185,16 +190,28 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[mt][v] = 0.f;
   float m_run = -INFINITY, l_run = 0.f;
+  // MODS, where the registers suffice: the sums of the weights come from the matrix cores (a V^T
+  // fragment of ones), of the same rounded weights that the output is made of
+  constexpr bool MFMA_SUM = MODS && HEAD_DIM <= 64;
+  f32x16_t o_sum;
+#pragma unroll
+  for (int v = 0; v < 16; ++v) o_sum[v] = 0.f;
+  const bf16x8_t ones = as_frag((u32x4_t){0x3F803F80u, 0x3F803F80u, 0x3F803F80u, 0x3F803F80u});
   // (with MODS the scores are scaled, worked on and brought to units of log 2 one by one)
   const float sc = MODS ? 1.0f : scale * LOG2E;
-  __shared__ float sh_bias[MODS ? P_BIAS_MAX : 1];
+  // the head's biases in units of log 2, the far ones first, with room for the distances that only
+  // masked scores and the block's spread of rows reach: place bias_top - dist
+  __shared__ float sh_bias[MODS ? P_BIAS_MAX + 2 * P_BIAS_EDGE : 1];
   const bool has_bias = MODS && mods.dist_bias != nullptr;
   const bool bias_in_lds = has_bias && mods.dist_cols <= P_BIAS_MAX;
-  const float* bias_row = has_bias ? mods.dist_bias + (size_t)h * mods.dist_cols : nullptr;
-  const float far_bias = has_bias ? bias_row[mods.dist_cols - 1] : 0.f;
+  const float* bias_row = has_bias ? kappai_bias_row(mods, h) : nullptr;
+  const float far_bias = has_bias ? bias_row[mods.dist_cols - 1] * LOG2E : 0.f;
+  const int bias_top = MODS ? mods.dist_cols - 1 + P_BIAS_EDGE : 0;
+  const int bias_pos = row_ok ? my_pos : pos_first;
   if (MODS) {
     if (bias_in_lds)
-      for (int i = threadIdx.x; i < mods.dist_cols; i += P_NW * WAVE) sh_bias[i] = bias_row[i];
+      for (int i = threadIdx.x; i < mods.dist_cols + 2 * P_BIAS_EDGE; i += P_NW * WAVE)
+        sh_bias[i] = bias_row[max(0, min(bias_top - i, mods.dist_cols - 1))] * LOG2E;
     __syncthreads();
   }
 
@@ -276,21 +293,24 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
     // lane holds, for query `col`, keys kb + 8*(v/4) + 4*hh + v%4
     if (MODS) {
       const bool capped = mods.softcap > 0.f;
-      const bool far = has_bias && pos_first - (kb + 31) >= mods.dist_cols - 1;
+      const float by = capped ? LOG2E : scale * LOG2E;
+      if (capped)
 #pragma unroll
-      for (int v = 0; v < 16; ++v) {
-        float x = s[v] * scale;
-        if (capped) x = kappai_fast_cap(x, mods.softcap);
-        if (has_bias) {
-          if (far) {
-            x += far_bias;
-          } else {
-            const int key = kb + 8 * (v / 4) + 4 * hh + v % 4;
-            const int dist = max(0, min(my_pos - key, mods.dist_cols - 1));
-            x += bias_in_lds ? sh_bias[dist] : bias_row[dist];
-          }
+        for (int v = 0; v < 16; ++v) s[v] = kappai_fast_cap(s[v] * scale, mods.softcap);
+      if (!has_bias || pos_first - (kb + 31) >= mods.dist_cols - 1) {
+#pragma unroll
+        for (int v = 0; v < 16; ++v) s[v] = fmaf(s[v], by, far_bias);
+      } else if (bias_in_lds) {
+        // (a distance here is at most dist_cols - 2 + 62 and at least -62)
+        const float* at0 = sh_bias + (bias_top - (bias_pos - kb - 4 * hh));
+#pragma unroll
+        for (int v = 0; v < 16; ++v) s[v] = fmaf(s[v], by, at0[8 * (v / 4) + v % 4]);
+      } else {
+#pragma unroll
+        for (int v = 0; v < 16; ++v) {
+          const int dist = bias_pos - (kb + 8 * (v / 4) + 4 * hh + v % 4);
+          s[v] = fmaf(s[v], by, bias_row[max(0, min(dist, mods.dist_cols - 1))] * LOG2E);
         }
-        s[v] = x * LOG2E;
       }
     }
     float mloc = -INFINITY;
@@ -308,22 +328,33 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
       }
     }
     mloc = fmaxf(mloc, other_half(mloc));
-    const float m_new = fmaxf(m_run, mloc);
-    const float m_safe = m_new == -INFINITY ? 0.f : m_new;
-    const float corr = fast_exp2(m_run - m_safe);
+    // MODS: the reference that the weights are taken against moves only when a tile's maximum lies
+    // more than 2^8 above it (or there is none yet): most tiles leave the output accumulators alone
+    const bool move = !MODS || mloc > m_run + 8.0f;
+    if (!MODS || __builtin_amdgcn_ballot_w64(move) != 0) {
+      const float m_new = move ? fmaxf(m_run, mloc) : m_run;
+      const float corr = move ? fast_exp2(m_run - (m_new == -INFINITY ? 0.f : m_new)) : 1.0f;
+      l_run *= corr;
+      if (MFMA_SUM)
+#pragma unroll
+        for (int v = 0; v < 16; ++v) o_sum[v] *= corr;
+#pragma unroll
+      for (int mt = 0; mt < P_MT; ++mt)
+#pragma unroll
+        for (int v = 0; v < 16; ++v) o[mt][v] *= corr;
+      m_run = m_new;
+    }
+    const float m_safe = m_run == -INFINITY ? 0.f : m_run;
     float lsum = 0.f;
 #pragma unroll
     for (int v = 0; v < 16; ++v) {
       s[v] = fast_exp2(fmaf(s[v], sc, -m_safe));
-      lsum += s[v];
+      if (!MFMA_SUM) lsum += s[v];
     }
-    lsum += other_half(lsum);
-    l_run = l_run * corr + lsum;
-    m_run = m_new;
-#pragma unroll
-    for (int mt = 0; mt < P_MT; ++mt)
-#pragma unroll
-      for (int v = 0; v < 16; ++v) o[mt][v] *= corr;
+    if (!MFMA_SUM) {
+      lsum += other_half(lsum);
+      l_run += lsum;
+    }
     // ---- O^T += V^T P^T, two k-steps of 16 keys ---------------------------------------
 #pragma unroll
     for (int st = 0; st < 2; ++st) {
@@ -332,6 +363,7 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
                           pack_bf16(s[8 * st + 4], s[8 * st + 5]),
                           pack_bf16(s[8 * st + 6], s[8 * st + 7])};
       const bf16x8_t pf = as_frag(pw);
+      if (MFMA_SUM) o_sum = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ones, pf, o_sum, 0, 0, 0);
 #pragma unroll
       for (int mt = 0; mt < P_MT; ++mt) {
         const u32x4_t vw = {vfa[buf][st][mt].x, vfa[buf][st][mt].y, vfb[buf][st][mt].x,
@@ -360,6 +392,7 @@ __global__ __launch_bounds__(P_NW * WAVE) void attn_prefill_kernel(
       work(0, at(kb));
     }
   }
+  if (MFMA_SUM) l_run = o_sum[0];
   if (P_NW > 1) {
     // merge: every wave rescales to the common maximum; waves 1.. hand their sums to wave 0
     __shared__ float sh_m[P_NW][32], sh_l[P_NW][32];
@@ -1023,7 +1056,9 @@ __device__ __forceinline__ void attn_decode_wave(
   struct Chunk {
     u32x4_t kf[NCH][2][D_KS];
     u32x4_t vv[NCH][D_MT];
+    float bias[MODS ? NCH : 1][8];     // of the lane's eight keys, the last key first
   };
+  const float* bias_row = MODS && mods->dist_bias != nullptr ? kappai_bias_row(*mods, h) : nullptr;
   auto ask = [&](int c0, int my_page, Chunk& ch) {
     const int first_page = c0 / ps;
     // Row r of the key tile tt (of the 32 keys from kb) is key kb + 8 (r / 4) + 4 tt + r % 4:
@@ -1051,6 +1086,21 @@ __device__ __forceinline__ void attn_decode_wave(
       for (int mt = 0; mt < D_MT; ++mt)
         ch.vv[c][mt] = load_vt8_pg(vt_pool, pv, G, g, ps, 16 * mt + col, kb + 8 * kg,
                                     f_lo, f_hi);
+      if (MODS) {
+        if (bias_row != nullptr) {     // distances base .. base + 7, by the row's edges at most
+          const int base = max(-KAPPAI_BIAS_PAD, min(pos - kb - 8 * kg - 7, mods->dist_cols - 1));
+          const f32x4_any_t b0 = *reinterpret_cast<const f32x4_any_t*>(bias_row + base);
+          const f32x4_any_t b1 = *reinterpret_cast<const f32x4_any_t*>(bias_row + base + 4);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            ch.bias[c][i] = b0[i];
+            ch.bias[c][4 + i] = b1[i];
+          }
+        } else {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) ch.bias[c][i] = 0.f;
+        }
+      }
     }
   };
   // the pools do not hold the row's own key and value yet (or only just): the chunk that holds
@@ -1107,9 +1157,7 @@ __device__ __forceinline__ void attn_decode_wave(
           if (MODS) {
             float x = s[tt][v] * scale;
             if (mods->softcap > 0.f) x = kappai_fast_cap(x, mods->softcap);
-            if (mods->dist_bias != nullptr)
-              x += mods->dist_bias[(size_t)h * mods->dist_cols +
-                                   max(0, min(pos - key, mods->dist_cols - 1))];
+            x += ch.bias[c][7 - (4 * tt + v)];
             s[tt][v] = ok ? x * LOG2E : -INFINITY;
           }
           else

@@ -214,38 +214,41 @@ extern "C" int kappai_moe_route_squashed(const void* x, int ldx, int x_is_bf16,
 }
 
 // The pairs sorted by expert, stably and without atomics.  The waves of one block each take a
-// run of the pairs, 64 at a time: the lanes with the same expert are found by ballots and placed
-// by counting the lanes below.  Pass 1 counts per wave and expert; then every expert's run gets
-// its first slot (a multiple of MOE_TILE_M) and every wave its place in the run; pass 2 places.
+// run of the pairs, 64 at a time: a lane finds the lanes with its own expert by one ballot a bit of
+// the expert's number and its place among them by counting those below.  Pass 1 counts per wave
+// and expert; then every expert's run gets its first slot (a multiple of MOE_TILE_M) and every
+// wave its place in the run; pass 2 places.
 #define MOE_PLAN_MAX_WAVES 16
 
 __device__ __forceinline__ void moe_plan_pass(const int* __restrict__ idx, int p_lo, int p_hi,
-                                              int* cnt, const int* start, bool place,
+                                              int n_bits, int* cnt, const int* start, bool place,
                                               int* __restrict__ slot_of_pair,
                                               int* __restrict__ pair_of_slot) {
   const int lane = threadIdx.x % WAVE;
+  int next = p_lo + lane < p_hi ? idx[p_lo + lane] : 0;
   for (int p0 = p_lo; p0 < p_hi; p0 += WAVE) {
-    const int p = p0 + lane;
-    const int e = p < p_hi ? idx[p] : -1;
-    bool todo = p < p_hi;
-    while (true) {
-      const unsigned long long rest = __ballot(todo);
-      if (!rest) break;
-      const int cur = __shfl(e, __ffsll((long long)rest) - 1);
-      const bool mine = todo && e == cur;
-      const unsigned long long mask = __ballot(mine);
-      const int before = cnt[cur];          // (only this wave writes its counters)
-      if (place && mine) {
-        const int slot = start[cur] + before + __popcll(mask & ((1ull << lane) - 1ull));
-        slot_of_pair[p] = slot;
-        pair_of_slot[slot] = p;
-      }
-      __builtin_amdgcn_wave_barrier();
-      if (lane == 0) cnt[cur] = before + __popcll(mask);
-      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-      __builtin_amdgcn_wave_barrier();
-      if (mine) todo = false;
+    const int p = p0 + lane, e = next;
+    const bool mine = p < p_hi;
+    next = p + WAVE < p_hi ? idx[p + WAVE] : 0;
+    unsigned long long same = __ballot(mine);
+    for (int b = 0; b < n_bits; ++b) {
+      const bool one = (e >> b) & 1;
+      const unsigned long long ones = __ballot(one);
+      same &= one ? ones : ~ones;
     }
+    // (only this wave writes its counters; lanes of different experts write different ones)
+    const int before = mine ? cnt[e] : 0;
+    if (place && mine) {
+      const int slot = start[e] + before + __popcll(same & ((1ull << lane) - 1ull));
+      slot_of_pair[p] = slot;
+      pair_of_slot[slot] = p;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    if (mine && lane == __ffsll((long long)same) - 1) cnt[e] = before + __popcll(same);
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
 }
 
@@ -266,7 +269,8 @@ __global__ __launch_bounds__(MOE_PLAN_MAX_WAVES * WAVE) void moe_plan_kernel(
   __syncthreads();
   const int per = ((P + n_waves * WAVE - 1) / (n_waves * WAVE)) * WAVE;
   const int p_lo = min(P, wave * per), p_hi = min(P, p_lo + per);
-  moe_plan_pass(idx, p_lo, p_hi, cnt + wave * E, nullptr, false, slot_of_pair, pair_of_slot);
+  const int n_bits = E > 1 ? 32 - __clz(E - 1) : 0;
+  moe_plan_pass(idx, p_lo, p_hi, n_bits, cnt + wave * E, nullptr, false, slot_of_pair, pair_of_slot);
   __syncthreads();
   // the runs' lengths and, inside a run, the waves one after the other
   for (int e = tid; e < E; e += nt) {
@@ -295,7 +299,7 @@ __global__ __launch_bounds__(MOE_PLAN_MAX_WAVES * WAVE) void moe_plan_kernel(
     for (int i = 0; i < n; ++i) tile_expert[first / MOE_TILE_M + i] = e;
   }
   __syncthreads();
-  moe_plan_pass(idx, p_lo, p_hi, cnt + wave * E, start + wave * E, true, slot_of_pair,
+  moe_plan_pass(idx, p_lo, p_hi, n_bits, cnt + wave * E, start + wave * E, true, slot_of_pair,
                 pair_of_slot);
 }
 

@@ -2,7 +2,10 @@
 // sink: one more term of the softmax's denominator that has no key and no value.
 //   softcap     0: nothing; else score <- softcap * tanh(score / softcap)
 //   dist_bias   [heads, dist_cols] float32, added after the cap: column min(i - j, dist_cols - 1)
-//               for query position i and key position j; null: nothing
+//               for query position i and key position j; null: nothing.  In memory a head's row
+//               has KAPPAI_BIAS_PAD more columns on either side (zeros in front, the last column
+//               repeated behind), so that the biases of eight keys in a row are eight neighbours
+//               wherever the row begins or ends
 //   sink        [heads] float32: exp(sink[h]) joins the denominator once; null: nothing
 //   keep_first  the first keep_first positions of a sequence are seen by every later one, whatever
 //               the window or chunk; 0: nothing is kept
@@ -18,6 +21,8 @@ __host__ __device__ __forceinline__ int kappai_first_key(int pos, int window) {
   if (window < 0) return pos < 0 ? 0 : pos - pos % (-window);
   return 0;
 }
+
+#define KAPPAI_BIAS_PAD 8
 
 struct kappai_score_mods {
   float softcap;
@@ -50,6 +55,10 @@ __host__ __device__ __forceinline__ bool kappai_mods_change_scores(const kappai_
   return m != nullptr && (m->softcap > 0.f || m->dist_bias != nullptr || m->keep_first > 0);
 }
 
+__device__ __forceinline__ const float* kappai_bias_row(const kappai_score_mods& m, int h) {
+  return m.dist_bias + (size_t)h * (m.dist_cols + 2 * KAPPAI_BIAS_PAD) + KAPPAI_BIAS_PAD;
+}
+
 // cap * tanh(s / cap) for the kernels that work in bfloat16: tanh(x) = 1 - 2 / (1 + e^(2x)) by the
 // hardware's exponential and reciprocal (absolute error of a few 1e-7 of the cap).
 __device__ __forceinline__ float kappai_fast_cap(float s, float cap) {
@@ -62,6 +71,6 @@ __device__ __forceinline__ float kappai_modified_score(const kappai_score_mods& 
                                                        int dist) {
   if (m.softcap > 0.f) s = m.softcap * tanhf(s / m.softcap);
   if (m.dist_bias != nullptr)
-    s += m.dist_bias[(size_t)h * m.dist_cols + max(0, min(dist, m.dist_cols - 1))];
+    s += kappai_bias_row(m, h)[max(0, min(dist, m.dist_cols - 1))];
   return s;
 }

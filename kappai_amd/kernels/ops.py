@@ -819,6 +819,9 @@ def qk_norm_rope_store(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_di
     return qkv if parts is None else q_out
 
 
+BIAS_PAD = 8       # columns on either side of a head's row of distance biases (csrc/score_mods.h)
+
+
 class ScoreModsC(ctypes.Structure):
     """``kappai_score_mods`` of csrc/score_mods.h."""
     _fields_ = [("softcap", _c_float), ("dist_bias", _vp), ("dist_cols", _c_int), ("sink", _vp),
@@ -838,6 +841,15 @@ class ScoreMods:
     sink: Optional[torch.Tensor] = None
     keep_first: int = 0
 
+    def __post_init__(self):
+        padded = None
+        if self.distance_bias is not None and self.distance_bias.dim() == 2 \
+                and self.distance_bias.shape[1]:
+            t = self.distance_bias                 # a row as the kernels read it
+            padded = torch.cat([torch.zeros_like(t[:, :1]).expand(-1, BIAS_PAD), t,
+                                t[:, -1:].expand(-1, BIAS_PAD)], dim=1).contiguous()
+        object.__setattr__(self, "_padded", padded)
+
     def active(self) -> bool:
         return (self.softcap > 0.0 or self.distance_bias is not None or self.sink is not None
                 or self.keep_first > 0)
@@ -855,7 +867,7 @@ class ScoreMods:
             _need(self.sink.shape == (n_heads,), lambda: f"sink {tuple(self.sink.shape)}")
         _need(self.keep_first >= 0, lambda: f"keep_first {self.keep_first}")
         return ScoreModsC(float(self.softcap),
-                          0 if self.distance_bias is None else self.distance_bias.data_ptr(), cols,
+                          0 if self._padded is None else self._padded.data_ptr(), cols,
                           0 if self.sink is None else self.sink.data_ptr(), int(self.keep_first))
 
 
