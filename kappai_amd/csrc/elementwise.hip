@@ -309,6 +309,175 @@ extern "C" int kappai_tanh_norm_step(float* resid, const void* y, int y_is_bf16,
 }
 
 // ---------------------------------------------------------------------------------------
+// RMS norms n(x) = x / sqrt(mean(x^2) + eps) * w on both sides of a sublayer in one pass over the
+// stream: resid += n_post(y), rows = n_pre(resid).  A block a row; the row stays in registers from
+// the loads over both sums of squares to the stores.  y comes as
+//   rows (float32 or bfloat16), or float planes [parts][T][D] that are added in order, or, with
+//   slot_of_pair, as a mixture's experts left it: also[t] * gate[t] first (what every row gets: rows
+//   or planes; a gate or none), then the sum over the row's `top` choices of wts[t, k] * y[slot of
+//   (t, k)], in the order of k; slot -1 stands for the row x[t] itself.
+// post_w null: y is added as it is; pre_w null: no rows are wanted.  `pick`: only these rows are
+// normalised, and the stream keeps its old values.  Everything in float32.
+// ---------------------------------------------------------------------------------------
+struct kappai_update {
+  const void* y;
+  int y_is_bf16, parts;
+  const int* slot_of_pair;
+  const float* wts;
+  int top;
+  const void* also;
+  int also_is_bf16, also_parts;
+  const float* also_gate;
+  const void* x;
+  int ldx, x_is_bf16;
+};
+
+template <int VEC>
+__device__ __forceinline__ void load_cols(const void* p, int is_bf16, size_t at, float (&v)[VEC]) {
+  if (is_bf16) load_cols<VEC>((const bf16_t*)p + at, v);
+  else load_cols<VEC>((const float*)p + at, v);
+}
+
+// rows, or planes added in order
+template <int VEC>
+__device__ __forceinline__ void load_planes(const void* p, int is_bf16, int parts, size_t plane,
+                                            size_t at, float (&u)[VEC]) {
+  load_cols<VEC>(p, is_bf16, at, u);
+#pragma unroll 4
+  for (int k = 1; k < parts; ++k) {
+    float v[VEC];
+    load_cols<VEC>((const float*)p + k * plane + at, v);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) u[j] += v[j];
+  }
+}
+
+template <int VEC>
+__device__ __forceinline__ void load_update(const kappai_update& up, size_t t, int c, int D,
+                                            size_t plane, float (&u)[VEC]) {
+  if (up.slot_of_pair == nullptr) {
+    load_planes<VEC>(up.y, up.y_is_bf16, up.parts, plane, t * D + c, u);
+    return;
+  }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) u[j] = 0.f;
+  if (up.also != nullptr) {
+    load_planes<VEC>(up.also, up.also_is_bf16, up.also_parts, plane, t * D + c, u);
+    const float g = up.also_gate != nullptr ? up.also_gate[t] : 1.f;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) u[j] *= g;
+  }
+  float own[VEC];
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) own[j] = 0.f;
+  if (up.x != nullptr) load_cols<VEC>(up.x, up.x_is_bf16, t * up.ldx + c, own);
+#pragma unroll 4
+  for (int k = 0; k < up.top; ++k) {
+    const int slot = up.slot_of_pair[t * up.top + k];
+    const float f = up.wts[t * up.top + k];
+    float v[VEC];
+    if (slot >= 0) {
+      load_cols<VEC>((const float*)up.y + (size_t)slot * D + c, v);
+    } else {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] = own[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) u[j] = fmaf(f, v[j], u[j]);
+  }
+}
+
+// NC pieces of VEC columns a thread, a block's width apart
+template <int VEC, int NC>
+__global__ __launch_bounds__(1024) void rms_norm_step_kernel(
+    float* __restrict__ resid, const kappai_update up, size_t plane,
+    const float* __restrict__ post_w, float post_eps, const float* __restrict__ pre_w,
+    float pre_eps, const int* __restrict__ pick, int D, int store, void* __restrict__ rows,
+    int rows_is_bf16) {
+  __shared__ float red[16];
+  const size_t r = blockIdx.x;
+  const size_t t = pick != nullptr ? (size_t)pick[r] : r;
+  float x[NC][VEC], u[NC][VEC], w[NC][VEC];
+  float ss = 0.f;
+  const bool update = up.y != nullptr;
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[i][j] = u[i][j] = w[i][j] = 0.f;
+    if (c >= D) continue;
+    load_cols<VEC>(resid + t * D + c, x[i]);
+    if (update) {
+      if (post_w != nullptr) load_cols<VEC>(post_w + c, w[i]);
+      load_update<VEC>(up, t, c, D, plane, u[i]);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss = fmaf(u[i][j], u[i][j], ss);
+  }
+  if (update) {
+    float inv = 1.f;
+    if (post_w != nullptr) inv = 1.0f / sqrtf(block_sum(ss, red) / (float)D + post_eps);
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (i * blockDim.x + threadIdx.x) * VEC;
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[i][j] += post_w != nullptr ? u[i][j] * inv * w[i][j] : u[i][j];
+      if (store && c < D) store_cols<VEC>(resid + t * D + c, x[i]);
+    }
+  }
+  if (rows == nullptr) return;
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * VEC;
+    if (c < D) load_cols<VEC>(pre_w + c, w[i]);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss = fmaf(x[i][j], x[i][j], ss);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)D + pre_eps);
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * VEC;
+    if (c >= D) continue;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[i][j] = x[i][j] * inv * w[i][j];
+    if (rows_is_bf16) store_cols<VEC>((bf16_t*)rows + r * D + c, x[i]);
+    else store_cols<VEC>((float*)rows + r * D + c, x[i]);
+  }
+}
+
+extern "C" int kappai_rms_norm_step(
+    float* resid, const void* y, int y_is_bf16, int parts, const int* slot_of_pair,
+    const float* wts, int top, const void* also, int also_is_bf16, int also_parts,
+    const float* also_gate, const void* x, int ldx, int x_is_bf16, const float* post_w,
+    float post_eps, const float* pre_w, float pre_eps, const int* pick, int n_rows, int T, int D,
+    void* rows, int rows_is_bf16, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (D < 1 || D > 8192 || (y && parts < 1) || (y_is_bf16 && (parts != 1 || slot_of_pair)) ||
+      (slot_of_pair && (!y || !wts || top < 1)) || (rows && !pre_w) || (!pick && n_rows != T) ||
+      (also && (also_parts < 1 || (also_is_bf16 && also_parts != 1))) || (x && ldx < D))
+    return (int)hipErrorInvalidValue;
+  const kappai_update up{y, y_is_bf16, parts, slot_of_pair, wts, top, also, also_is_bf16,
+                         also_parts, also_gate, x, ldx, x_is_bf16};
+  const bool vec = D % 4 == 0 && ldx % 4 == 0 &&
+                   ((uintptr_t)resid | (uintptr_t)y | (uintptr_t)post_w | (uintptr_t)pre_w |
+                    (uintptr_t)rows | (uintptr_t)also | (uintptr_t)x) % 16 == 0;
+  const int pieces = vec ? D / 4 : D;
+  const int threads = pieces >= 1024 ? 1024 : (pieces + WAVE - 1) / WAVE * WAVE;
+#define KAPPAI_RMS_STEP(V, N)                                                                    \
+  hipLaunchKernelGGL((rms_norm_step_kernel<V, N>), dim3(n_rows), dim3(threads), 0, stream, resid, \
+                     up, (size_t)T * D, post_w, post_eps, pre_w, pre_eps, pick, D, pick ? 0 : 1,  \
+                     rows, rows_is_bf16)
+  if (vec) {
+    if (pieces <= 1024) KAPPAI_RMS_STEP(4, 1); else KAPPAI_RMS_STEP(4, 2);
+  } else {
+    if (pieces <= 1024) KAPPAI_RMS_STEP(1, 1); else KAPPAI_RMS_STEP(1, 8);
+  }
+#undef KAPPAI_RMS_STEP
+  KAPPAI_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------------
 // Two sublayers' results side by side, made one update of the stream in float32:
 // out = scale_a * n_a(a) + scale_b * n_b(b), with n(y) = y / sqrt(mean(y^2) + eps) * w when a
 // weight is given and y itself when not.  a, b [T, D] in float32 or bfloat16 (one dtype); a block
@@ -740,37 +909,55 @@ extern "C" int kappai_unary(const void* in, void* out, long n, int kind, int is_
 }
 
 // act(gate) * up with a choice of act: 0 silu, 1 the tanh form of gelu,
-// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))).
-template <typename T>
+// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), 2 the clamped gate: g = min(gate, limit),
+// u = clamp(up, -limit, limit), g sigmoid(slope g) (u + shift).
+struct kappai_clamp { float limit, slope, shift; };
+
+__device__ __forceinline__ float glu_value(float g, float u, int kind, const kappai_clamp& c) {
+  if (kind == 2) {
+    g = fminf(g, c.limit);
+    u = fminf(fmaxf(u, -c.limit), c.limit);
+    return g / (1.0f + expf(-c.slope * g)) * (u + c.shift);
+  }
+  if (kind == 1)
+    return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+  return g / (1.0f + expf(-g)) * u;
+}
+
+// VEC columns a thread (4: F a multiple of four and 16-byte aligned pointers)
+template <typename T, int VEC>
 __global__ void glu_kernel(const T* __restrict__ gu, T* __restrict__ act, int F, size_t n,
-                           int kind) {
-  size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+                           int kind, kappai_clamp clamp) {
+  const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
   if (i >= n) return;
   const size_t t = i / F;
   const int f = (int)(i - t * F);
-  const float g = to_f32(gu[t * 2 * F + f]);
-  const float u = to_f32(gu[t * 2 * F + F + f]);
-  float a;
-  if (kind == 1)
-    a = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  else
-    a = g / (1.0f + expf(-g));
-  from_f32(act + i, a * u);
+  float g[VEC], u[VEC];
+  load_cols<VEC>(gu + t * 2 * F + f, g);
+  load_cols<VEC>(gu + t * 2 * F + F + f, u);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) g[j] = glu_value(g[j], u[j], kind, clamp);
+  store_cols<VEC>(act + i, g);
 }
 
 extern "C" int kappai_glu(const void* gu, void* act, int T, int F, int is_bf16, int kind,
-                          hipStream_t stream) {
+                          float limit, float slope, float shift, hipStream_t stream) {
   const size_t n = (size_t)T * F;
   if (n == 0) return 0;
-  if (kind < 0 || kind > 1) return (int)hipErrorInvalidValue;
+  if (kind < 0 || kind > 2) return (int)hipErrorInvalidValue;
+  const kappai_clamp clamp{limit, slope, shift};
+  const int vec = F % 4 == 0 && ((uintptr_t)gu | (uintptr_t)act) % 16 == 0 ? 4 : 1;
   const int threads = 256;
-  const unsigned blocks = (unsigned)((n + threads - 1) / threads);
-  if (is_bf16)
-    hipLaunchKernelGGL(glu_kernel<bf16_t>, dim3(blocks), dim3(threads), 0, stream,
-                       (const bf16_t*)gu, (bf16_t*)act, F, n, kind);
-  else
-    hipLaunchKernelGGL(glu_kernel<float>, dim3(blocks), dim3(threads), 0, stream,
-                       (const float*)gu, (float*)act, F, n, kind);
+  const unsigned blocks = (unsigned)((n / vec + threads - 1) / threads);
+#define KAPPAI_GLU(TT, V)                                                                        \
+  hipLaunchKernelGGL((glu_kernel<TT, V>), dim3(blocks), dim3(threads), 0, stream, (const TT*)gu, \
+                     (TT*)act, F, n, kind, clamp)
+  if (is_bf16) {
+    if (vec == 4) KAPPAI_GLU(bf16_t, 4); else KAPPAI_GLU(bf16_t, 1);
+  } else {
+    if (vec == 4) KAPPAI_GLU(float, 4); else KAPPAI_GLU(float, 1);
+  }
+#undef KAPPAI_GLU
   KAPPAI_RETURN_LAUNCH_STATUS();
 }
 

@@ -13,13 +13,9 @@
 // partial dot products meet by lane exchanges.  Tokens of a segment are walked in order; a
 // segment that starts at position 0 starts from zero, whatever the slot holds.
 #include "common.h"
+#include "matrix_state.h"
 
 #define LA_THREADS 256
-
-__device__ __forceinline__ float la_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
-__device__ __forceinline__ float la_softplus(float x) {
-  return x > 20.f ? x : log1pf(expf(x));
-}
 
 // ---------------------------------------------------------------------------------------
 // Short causal convolution per channel, then SiLU (act 1) or nothing (act 0), with an optional
@@ -88,6 +84,101 @@ __global__ __launch_bounds__(LA_THREADS) void conv_state_kernel(
   for (int i = 0; i < keep; ++i) st[(size_t)i * C] = kept[i];
 }
 
+// The same for bfloat16 with up to four taps: a thread makes CONV_ROWS neighbouring rows of eight
+// channels from one read of each input row (16-byte loads and stores).  C and the row stride are
+// multiples of eight, the pointers of 16 bytes.
+#define CONV_ROWS 4
+template <int NT>
+__global__ __launch_bounds__(LA_THREADS) void conv_silu_vec_kernel(
+    const bf16_t* __restrict__ x, int x_stride, const float* __restrict__ taps,
+    const float* __restrict__ state, const int* __restrict__ row_pos,
+    const int* __restrict__ row_seg, const int* __restrict__ seg_start,
+    const int* __restrict__ seg_slot, int T, int C, const float* __restrict__ bias, int act,
+    bf16_t* __restrict__ out) {
+  const int t0 = blockIdx.x * CONV_ROWS;
+  const int c = (blockIdx.y * LA_THREADS + threadIdx.x) * 8;
+  if (c >= C) return;
+  uint4 in[CONV_ROWS + NT - 1];
+#pragma unroll
+  for (int k = 0; k < CONV_ROWS + NT - 1; ++k) {
+    const int t = min(max(t0 - (NT - 1) + k, 0), T - 1);
+    in[k] = *reinterpret_cast<const uint4*>(x + (size_t)t * x_stride + c);
+  }
+  float w[NT][8], tp[8 * NT], b8[8];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) load8(taps + (size_t)c * NT + 8 * j, tp + 8 * j);
+#pragma unroll
+  for (int j = 0; j < NT; ++j)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) w[j][e] = tp[e * NT + j];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) b8[e] = 0.f;
+  if (bias != nullptr) load8(bias + c, b8);
+#pragma unroll
+  for (int r = 0; r < CONV_ROWS; ++r) {
+    const int t = t0 + r;
+    if (t >= T) break;
+    const int seg = row_seg[t], first = seg_start[seg], pos = row_pos[t];
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = 0.f;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      const int back = NT - 1 - j;
+      float v[8];
+      if (t - back >= first) {
+        const uint32_t q[4] = {in[r + j].x, in[r + j].y, in[r + j].z, in[r + j].w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          v[2 * i] = __uint_as_float(q[i] << 16);
+          v[2 * i + 1] = __uint_as_float(q[i] & 0xffff0000u);
+        }
+      } else if (back <= pos) {
+        load8(state + ((size_t)seg_slot[seg] * (NT - 1) + (NT - 1 - (back - (t - first)))) * C + c,
+              v);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = 0.f;
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[e] = fmaf(w[j][e], v[e], acc[e]);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      acc[e] += b8[e];
+      if (act) acc[e] *= la_sigmoid(acc[e]);
+    }
+    store8(out + (size_t)t * C + c, acc);
+  }
+}
+
+// A step of single rows: output and history of a channel by one thread.
+template <typename T>
+__global__ __launch_bounds__(LA_THREADS) void conv_silu_step_kernel(
+    const T* __restrict__ x, int x_stride, const float* __restrict__ taps, int n_taps,
+    float* __restrict__ state, const int* __restrict__ row_pos,
+    const int* __restrict__ seg_slot, int C, const float* __restrict__ bias, int act,
+    T* __restrict__ out) {
+  const int t = blockIdx.x;
+  const int c = blockIdx.y * LA_THREADS + threadIdx.x;
+  if (c >= C) return;
+  const int pos = row_pos[t], keep = n_taps - 1;
+  float* st = state + (size_t)seg_slot[t] * keep * C + c;
+  const float cur = to_f32(x[(size_t)t * x_stride + c]);
+  const float* tc = taps + (size_t)c * n_taps;
+  float acc = 0.f;
+  for (int i = 0; i < keep; ++i) {
+    // entry i is the input keep - i tokens before this one (nothing before position 0)
+    const float v = keep - i <= pos ? st[(size_t)i * C] : 0.f;
+    acc = fmaf(tc[i], v, acc);
+    if (i > 0) st[(size_t)(i - 1) * C] = v;
+  }
+  if (keep > 0) st[(size_t)(keep - 1) * C] = cur;
+  acc = fmaf(tc[keep], cur, acc);
+  if (bias != nullptr) acc += bias[c];
+  from_f32(out + (size_t)t * C + c, act ? acc * la_sigmoid(acc) : acc);
+}
+
 extern "C" int kappai_conv_silu(const void* x, int x_stride, const float* taps, int n_taps,
                                 float* state, const int* row_pos, const int* row_seg,
                                 const int* seg_start, const int* seg_pos0, const int* seg_slot,
@@ -96,7 +187,38 @@ extern "C" int kappai_conv_silu(const void* x, int x_stride, const float* taps, 
   if (T <= 0 || S <= 0) return 0;
   if (n_taps < 1 || n_taps > 17 || S > 65535 || C > 65535 * LA_THREADS) return (int)hipErrorInvalidValue;
   const int bx = (C + LA_THREADS - 1) / LA_THREADS;
-  if (is_bf16) {
+  if (T == S) {                       // (no segment is empty: single rows)
+    if (is_bf16)
+      hipLaunchKernelGGL(conv_silu_step_kernel<bf16_t>, dim3(T, bx), dim3(LA_THREADS), 0, stream,
+                         (const bf16_t*)x, x_stride, taps, n_taps, state, row_pos, seg_slot, C,
+                         bias, act, (bf16_t*)out);
+    else
+      hipLaunchKernelGGL(conv_silu_step_kernel<float>, dim3(T, bx), dim3(LA_THREADS), 0, stream,
+                         (const float*)x, x_stride, taps, n_taps, state, row_pos, seg_slot, C,
+                         bias, act, (float*)out);
+    KAPPAI_RETURN_LAUNCH_STATUS();
+  }
+  const bool vec = is_bf16 && n_taps <= 4 && C % 8 == 0 && x_stride % 8 == 0 &&
+                   ((uintptr_t)x | (uintptr_t)taps | (uintptr_t)state | (uintptr_t)bias |
+                    (uintptr_t)out) % 16 == 0;
+  if (vec) {
+    const dim3 grid((T + CONV_ROWS - 1) / CONV_ROWS, (C / 8 + LA_THREADS - 1) / LA_THREADS);
+#define CONV_VEC(N)                                                                              \
+  hipLaunchKernelGGL(conv_silu_vec_kernel<N>, grid, dim3(LA_THREADS), 0, stream,                 \
+                     (const bf16_t*)x, x_stride, taps, state, row_pos, row_seg, seg_start,       \
+                     seg_slot, T, C, bias, act, (bf16_t*)out)
+    switch (n_taps) {
+      case 1: CONV_VEC(1); break;
+      case 2: CONV_VEC(2); break;
+      case 3: CONV_VEC(3); break;
+      default: CONV_VEC(4); break;
+    }
+#undef CONV_VEC
+    if (n_taps > 1)
+      hipLaunchKernelGGL(conv_state_kernel<bf16_t>, dim3(bx, S), dim3(LA_THREADS), 0, stream,
+                         (const bf16_t*)x, x_stride, n_taps, state, seg_start, seg_pos0, seg_slot,
+                         C);
+  } else if (is_bf16) {
     hipLaunchKernelGGL(conv_silu_kernel<bf16_t>, dim3(T, bx), dim3(LA_THREADS), 0, stream,
                        (const bf16_t*)x, x_stride, taps, n_taps, state, row_pos, row_seg,
                        seg_start, seg_slot, C, bias, act, (bf16_t*)out);
@@ -299,61 +421,6 @@ extern "C" int kappai_recurrence_prep(const void* q, int q_stride, const void* k
 // ---------------------------------------------------------------------------------------
 #define LA_MAX_WAVES 4
 #define LA_MAX_CHUNK 16
-
-// the r-th of a lane's rows
-template <int KS>
-__device__ __forceinline__ int la_row(int s, int r) { return 4 * ((r / 4) * KS + s) + r % 4; }
-
-template <int KS>
-__device__ __forceinline__ float ks_sum(float v) {
-  if (KS >= 2) v += dpp_move<0xB1>(v);      // quad_perm [1, 0, 3, 2]
-  if (KS >= 4) v += dpp_move<0x4E>(v);      // quad_perm [2, 3, 0, 1]
-  if (KS >= 8) v += dpp_move<0x141>(v);     // the other quad of a half row (row_half_mirror)
-  if (KS >= 16) v += dpp_move<0x140>(v);    // the other half of a row (row_mirror)
-  if (KS >= 32) v += lane_xor16(v);
-  if (KS >= 64) v += lane_xor32(v);
-  return v;
-}
-
-template <int KS, int R>
-__device__ __forceinline__ void la_load_rows(const float* __restrict__ st, int s, int d,
-                                             bool carry, float (&S)[R]) {
-#pragma unroll
-  for (int r = 0; r < R; ++r) S[r] = 0.f;
-  if (!carry) return;
-  if (d % 4 == 0) {
-#pragma unroll
-    for (int r4 = 0; r4 < R; r4 += 4) {
-      const int row = la_row<KS>(s, r4);
-      if (row < d) {
-        const float4 x = *reinterpret_cast<const float4*>(st + row);
-        S[r4] = x.x; S[r4 + 1] = x.y; S[r4 + 2] = x.z; S[r4 + 3] = x.w;
-      }
-    }
-  } else {
-#pragma unroll
-    for (int r = 0; r < R; ++r)
-      if (la_row<KS>(s, r) < d) S[r] = st[la_row<KS>(s, r)];
-  }
-}
-
-template <int KS, int R>
-__device__ __forceinline__ void la_store_rows(float* __restrict__ st, int s, int d,
-                                              const float (&S)[R]) {
-  if (d % 4 == 0) {
-#pragma unroll
-    for (int r4 = 0; r4 < R; r4 += 4) {
-      const int row = la_row<KS>(s, r4);
-      if (row < d)
-        *reinterpret_cast<float4*>(st + row) =
-            make_float4(S[r4], S[r4 + 1], S[r4 + 2], S[r4 + 3]);
-    }
-  } else {
-#pragma unroll
-    for (int r = 0; r < R; ++r)
-      if (la_row<KS>(s, r) < d) st[la_row<KS>(s, r)] = S[r];
-  }
-}
 
 // One token: S, the lane's rows of q, k and the decay, the column's v, the head's beta.  The dot
 // products are summed in four strands (rows r, r + 4, ...) that meet at the end: four short
@@ -1151,22 +1218,31 @@ extern "C" int kappai_channel_decay_chunks(const float* qf, const float* kf, con
 
 // ---------------------------------------------------------------------------------------
 // Per head: o / sqrt(mean(o^2) + eps) * weight[dv] * gate, gate = silu(g) (kind 0) or sigmoid(g)
-// (kind 1) of the projection g [T, >= H dv] with a row stride.  A wave a (row, head).
+// (kind 1) of the projection g [T, >= H dv] with a row stride; or, with `gate_first`, the same norm
+// of o * gate.  A wave a (row, head).
 // weight_stride: 0 when the heads share one weight [dv], dv when each has its own [H, dv].
 // ---------------------------------------------------------------------------------------
 #define HNG_WIDE_THREADS 256      // heads of more than 512 values take a block of four waves
 template <typename T>
 __global__ __launch_bounds__(HNG_WIDE_THREADS) void head_norm_gate_kernel(
     const float* __restrict__ o, const float* __restrict__ weight, float eps,
-    const T* __restrict__ g, int g_stride, int gate_kind, int H, int dv, int weight_stride,
-    T* __restrict__ out) {
+    const T* __restrict__ g, int g_stride, int gate_kind, int gate_first, int H, int dv,
+    int weight_stride, T* __restrict__ out) {
   __shared__ float part[HNG_WIDE_THREADS / WAVE];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int threads = blockDim.x;
   weight += (size_t)h * weight_stride;
   const float* orow = o + ((size_t)t * H + h) * dv;
+  const T* gr = g + (size_t)t * g_stride + (size_t)h * dv;
+  auto gate = [&](int e) -> float {
+    const float gv = to_f32(gr[e]);
+    return gate_kind == 0 ? gv * la_sigmoid(gv) : la_sigmoid(gv);
+  };
   float ss = 0.f;
-  for (int e = lane; e < dv; e += threads) ss = fmaf(orow[e], orow[e], ss);
+  for (int e = lane; e < dv; e += threads) {
+    const float v = gate_first ? orow[e] * gate(e) : orow[e];
+    ss = fmaf(v, v, ss);
+  }
   ss = wave_sum(ss);
   if (threads > WAVE) {
     if (lane % WAVE == 0) part[lane / WAVE] = ss;
@@ -1175,27 +1251,68 @@ __global__ __launch_bounds__(HNG_WIDE_THREADS) void head_norm_gate_kernel(
     for (int w = 0; w < threads / WAVE; ++w) ss += part[w];
   }
   const float inv = 1.0f / sqrtf(ss / (float)dv + eps);
-  const T* gr = g + (size_t)t * g_stride + (size_t)h * dv;
-  for (int e = lane; e < dv; e += threads) {
-    const float gv = to_f32(gr[e]);
-    const float gate = gate_kind == 0 ? gv * la_sigmoid(gv) : la_sigmoid(gv);
-    from_f32(out + ((size_t)t * H + h) * dv + e, orow[e] * inv * weight[e] * gate);
+  for (int e = lane; e < dv; e += threads)
+    from_f32(out + ((size_t)t * H + h) * dv + e, orow[e] * inv * weight[e] * gate(e));
+}
+
+// Wide heads (512 to 8192 values, a multiple of eight, 16-byte aligned rows): eight values a thread,
+// kept in registers between the sum of squares and the scaling.
+template <typename T>
+__global__ __launch_bounds__(1024) void head_norm_gate_vec_kernel(
+    const float* __restrict__ o, const float* __restrict__ weight, float eps,
+    const T* __restrict__ g, int g_stride, int gate_kind, int gate_first, int H, int dv,
+    int weight_stride, T* __restrict__ out) {
+  __shared__ float red[16];
+  const int t = blockIdx.x, h = blockIdx.y, e0 = threadIdx.x * 8;
+  const size_t at = ((size_t)t * H + h) * dv + e0;
+  float v[8], w[8], gate[8], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = w[i] = gate[i] = 0.f;
+  if (e0 < dv) {
+    load8(o + at, v);
+    load8(g + (size_t)t * g_stride + (size_t)h * dv + e0, gate);
+    load8(weight + (size_t)h * weight_stride + e0, w);
   }
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    gate[i] = gate_kind == 0 ? gate[i] * la_sigmoid(gate[i]) : la_sigmoid(gate[i]);
+    const float x = gate_first ? v[i] * gate[i] : v[i];
+    ss = fmaf(x, x, ss);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)dv + eps);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = v[i] * inv * w[i] * gate[i];
+  if (e0 < dv) store8(out + at, v);
 }
 
 extern "C" int kappai_head_norm_gate(const float* o, const float* weight, float eps, const void* g,
-                                     int g_stride, int gate_kind, int T, int H, int dv,
-                                     int weight_stride, void* out, int is_bf16,
+                                     int g_stride, int gate_kind, int gate_first, int T, int H,
+                                     int dv, int weight_stride, void* out, int is_bf16,
                                      hipStream_t stream) {
   if (T <= 0) return 0;
   if (H < 1 || H > 65535 || dv < 1 || gate_kind < 0 || gate_kind > 1)
     return (int)hipErrorInvalidValue;
+  if (dv >= 512 && dv <= 8192 && dv % 8 == 0 && g_stride % 8 == 0 && weight_stride % 4 == 0 &&
+      ((uintptr_t)o | (uintptr_t)weight | (uintptr_t)g | (uintptr_t)out) % 16 == 0) {
+    const dim3 wide((dv / 8 + WAVE - 1) / WAVE * WAVE);
+    if (is_bf16)
+      hipLaunchKernelGGL(head_norm_gate_vec_kernel<bf16_t>, dim3(T, H), wide, 0, stream, o,
+                         weight, eps, (const bf16_t*)g, g_stride, gate_kind, gate_first, H, dv,
+                         weight_stride, (bf16_t*)out);
+    else
+      hipLaunchKernelGGL(head_norm_gate_vec_kernel<float>, dim3(T, H), wide, 0, stream, o, weight,
+                         eps, (const float*)g, g_stride, gate_kind, gate_first, H, dv,
+                         weight_stride, (float*)out);
+    KAPPAI_RETURN_LAUNCH_STATUS();
+  }
   const dim3 block(dv > 512 ? HNG_WIDE_THREADS : WAVE);
   if (is_bf16)
     hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, dim3(T, H), block, 0, stream, o, weight,
-                       eps, (const bf16_t*)g, g_stride, gate_kind, H, dv, weight_stride, (bf16_t*)out);
+                       eps, (const bf16_t*)g, g_stride, gate_kind, gate_first, H, dv, weight_stride,
+                       (bf16_t*)out);
   else
     hipLaunchKernelGGL(head_norm_gate_kernel<float>, dim3(T, H), block, 0, stream, o, weight,
-                       eps, (const float*)g, g_stride, gate_kind, H, dv, weight_stride, (float*)out);
+                       eps, (const float*)g, g_stride, gate_kind, gate_first, H, dv, weight_stride,
+                       (float*)out);
   KAPPAI_RETURN_LAUNCH_STATUS();
 }

@@ -2,11 +2,13 @@
 // order, and the weighted sum.  Nothing is read back by the host: every launch is sized by the
 // number of rows alone, so a step with experts can be captured in a graph.
 //   moe_route     z = W_router h in float32, the `top` largest chosen (lowest index on ties),
-//                 weights = softmax over the chosen logits; or scores s = sigmoid(z), the choice by
-//                 s + a correction within the best groups of experts, weights = s times a constant
+//                 weights = softmax over the chosen logits; or scores s = sigmoid(z) or softmax(z),
+//                 the choice by s + a correction within the best groups of experts, weights = s
+//                 times a constant; and the gate of an expert that every row takes
 //   moe_plan      (row, choice) pairs in expert order, every expert's run starting on a tile of
-//                 MOE_TILE_M slots: slot_of_pair, pair_of_slot (-1: empty), tile_expert (-1: unused)
-//   moe_gemm      tile by tile: act = silu(x Wg^T) * (x Wu^T) on gathered rows, or y = act Wd^T
+//                 MOE_TILE_M slots: slot_of_pair, pair_of_slot (-1: empty), tile_expert (-1: unused);
+//                 pairs of experts that hand their input on (numbers >= E) get slot -1 and no place
+//   moe_gemm      tile by tile: act = gate(x Wg^T) * (x Wu^T) on gathered rows, or y = act Wd^T
 //   moe_combine   out[t] = sum_k weight[t, k] * y[slot of (t, k)], in the order of k, float32
 #include "common.h"
 
@@ -21,28 +23,38 @@ extern "C" int kappai_moe_tile_rows() { return MOE_TILE_M; }
 
 #define MOE_ROUTE_GROUP 16      // experts whose sums a thread carries side by side
 
-// How a router that squashes every logit by itself chooses: score s = sigmoid(z), choice score
-// s + correction[e] (null: s).  The experts form `groups` equal groups of neighbours; a group's
-// score is the sum of its two largest choice scores, and only experts of the `keep` best groups can
-// be chosen (groups 1: all of them).  The weight of a chosen expert is s * scale.
-struct moe_squashed_choice {
+// How a router that scores every expert chooses: score s = sigmoid(z) of its own logit (over_all
+// 0) or softmax(z) over all experts (1), choice score s + correction[e] (null: s).  The experts form
+// `groups` equal groups of neighbours; a group's worth is the sum of its two largest choice scores
+// (best 2) or the largest (1), and only experts of the `keep` best groups can be chosen (groups 1:
+// all of them).  The weight of a chosen expert is s * scale.
+struct moe_scored_choice {
   const float* correction;
-  int groups, keep;
+  int groups, keep, over_all, best;
   float scale;
 };
 
 // The choice scores of the row in `choice` [E] (logits on entry) and the scores in `score` [E]; one
 // wave.  `group_score`: LDS for `groups` floats.
-__device__ __forceinline__ void moe_squash(const moe_squashed_choice& c, int E, float* choice,
-                                           float* score, float* group_score) {
+__device__ __forceinline__ void moe_score(const moe_scored_choice& c, int E, float* choice,
+                                          float* score, float* group_score) {
   const int lane = threadIdx.x % WAVE;
   auto meet = [] {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   };
+  float top = 0.f, total = 1.f;
+  if (c.over_all) {
+    top = -INFINITY;
+    for (int e = lane; e < E; e += WAVE) top = fmaxf(top, choice[e]);
+    top = wave_max(top);
+    total = 0.f;
+    for (int e = lane; e < E; e += WAVE) total += expf(choice[e] - top);
+    total = wave_sum(total);
+  }
   for (int e = lane; e < E; e += WAVE) {
-    const float s = 1.0f / (1.0f + expf(-choice[e]));
+    const float s = c.over_all ? expf(choice[e] - top) / total : 1.0f / (1.0f + expf(-choice[e]));
     score[e] = s;
     choice[e] = c.correction ? s + c.correction[e] : s;
   }
@@ -56,7 +68,7 @@ __device__ __forceinline__ void moe_squash(const moe_squashed_choice& c, int E, 
       b = fmaxf(b, fminf(a, v));
       a = fmaxf(a, v);
     }
-    group_score[g] = size > 1 ? a + b : a;
+    group_score[g] = size > 1 && c.best == 2 ? a + b : a;
   }
   meet();
   for (int g = lane; g < c.groups; g += WAVE) {
@@ -73,20 +85,22 @@ __device__ __forceinline__ void moe_squash(const moe_squashed_choice& c, int E, 
 // A block a row.  The threads stride over the row four columns at a time (one column at a time
 // when the width or an address does not allow 16-byte loads), each with the sums of a group of
 // experts, whose loads are all asked for before the first is used; the waves' sums meet in LDS
-// and are added in the order of the waves.  Then the first wave chooses.
-template <typename T, int VEC, bool SQUASHED>
+// and are added in the order of the waves.  Then the first wave chooses.  `gates` (null: none): the
+// router holds one more row behind the E experts', and sigmoid of its logit is the row's gate.
+template <typename T, int VEC, bool SCORED>
 __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
     const T* __restrict__ x, int ldx, const float* __restrict__ router,
-    const float* __restrict__ bias, int n_rows, int D, int E, int top, moe_squashed_choice sq,
-    int* __restrict__ idx, float* __restrict__ wts) {
+    const float* __restrict__ bias, int n_rows, int D, int E, int top, moe_scored_choice sq,
+    float* __restrict__ gates, int* __restrict__ idx, float* __restrict__ wts) {
   extern __shared__ float route_lds[];
   constexpr int NW = MOE_THREADS / WAVE;
-  float* logits = route_lds;                       // [E]
-  float* part = route_lds + E;                     // [MOE_ROUTE_GROUP][NW]
+  const int n_logits = gates != nullptr ? E + 1 : E;
+  float* logits = route_lds;                       // [n_logits]
+  float* part = route_lds + n_logits;              // [MOE_ROUTE_GROUP][NW]
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int row = blockIdx.x;
   const T* xr = x + (size_t)row * ldx;
-  for (int e0 = 0; e0 < E; e0 += MOE_ROUTE_GROUP) {
+  for (int e0 = 0; e0 < n_logits; e0 += MOE_ROUTE_GROUP) {
     float acc[MOE_ROUTE_GROUP];
 #pragma unroll
     for (int j = 0; j < MOE_ROUTE_GROUP; ++j) acc[j] = 0.f;
@@ -94,7 +108,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
       float xv[VEC], rv[MOE_ROUTE_GROUP][VEC];
 #pragma unroll
       for (int j = 0; j < MOE_ROUTE_GROUP; ++j) {
-        const float* r = router + (size_t)min(e0 + j, E - 1) * D + c;
+        const float* r = router + (size_t)min(e0 + j, n_logits - 1) * D + c;
         if (VEC == 4) {
           const float4 v = *reinterpret_cast<const float4*>(r);
           rv[j][0] = v.x; rv[j][VEC > 1 ? 1 : 0] = v.y; rv[j][VEC > 2 ? 2 : 0] = v.z;
@@ -116,16 +130,17 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
       if (lane == 0) part[j * NW + wave] = sum;
     }
     __syncthreads();
-    if (threadIdx.x < MOE_ROUTE_GROUP && e0 + threadIdx.x < E) {
+    if (threadIdx.x < MOE_ROUTE_GROUP && e0 + threadIdx.x < n_logits) {
       float sum = part[threadIdx.x * NW];
       for (int w = 1; w < NW; ++w) sum += part[threadIdx.x * NW + w];
-      logits[e0 + threadIdx.x] = bias ? sum + bias[e0 + threadIdx.x] : sum;
+      logits[e0 + threadIdx.x] = bias && e0 + threadIdx.x < E ? sum + bias[e0 + threadIdx.x] : sum;
     }
     __syncthreads();
   }
   if (wave != 0) return;
-  float* score = part + MOE_ROUTE_GROUP * NW;      // [E], then [groups] (squashed scores only)
-  if (SQUASHED) moe_squash(sq, E, logits, score, score + E);
+  if (gates != nullptr && lane == 0) gates[row] = 1.0f / (1.0f + expf(-logits[E]));
+  float* score = part + MOE_ROUTE_GROUP * NW;      // [E], then [groups] (scored choice only)
+  if (SCORED) moe_score(sq, E, logits, score, score + E);
   float cv[MOE_MAX_TOP];
   int ci[MOE_MAX_TOP];
 #pragma unroll
@@ -148,7 +163,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
     }
   }
   if (lane == 0) {
-    if (SQUASHED) {
+    if (SCORED) {
 #pragma unroll
       for (int k = 0; k < MOE_MAX_TOP; ++k)
         if (k < top) {
@@ -172,21 +187,22 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
 }
 
 static int moe_route_launch(const void* x, int ldx, int x_is_bf16, const float* router,
-                            const float* bias, int T, int D, int E, int top, bool squashed,
-                            moe_squashed_choice sq, int* idx, float* wts, hipStream_t stream) {
+                            const float* bias, int T, int D, int E, int top, bool scored,
+                            moe_scored_choice sq, float* gates, int* idx, float* wts,
+                            hipStream_t stream) {
   if (T <= 0) return 0;
   if (top < 1 || top > MOE_MAX_TOP || top > E || E > 4096) return (int)hipErrorInvalidValue;
-  if (squashed && (sq.groups < 1 || sq.keep < 1 || sq.keep > sq.groups || E % sq.groups ||
-                   top > E / sq.groups * sq.keep))
+  if (scored && (sq.groups < 1 || sq.keep < 1 || sq.keep > sq.groups || E % sq.groups ||
+                 top > E / sq.groups * sq.keep || sq.best < 1 || sq.best > 2))
     return (int)hipErrorInvalidValue;
-  const size_t lds = ((size_t)E + MOE_ROUTE_GROUP * (MOE_THREADS / WAVE) +
-                      (squashed ? E + sq.groups : 0)) * sizeof(float);
+  const size_t lds = ((size_t)E + 1 + MOE_ROUTE_GROUP * (MOE_THREADS / WAVE) +
+                      (scored ? E + sq.groups : 0)) * sizeof(float);
   const bool vec = D % 4 == 0 && (uintptr_t)router % 16 == 0;
 #define MOE_ROUTE_LAUNCH(TT, V)                                                                 \
-  if (squashed) MOE_ROUTE_LAUNCH_AS(TT, V, true); else MOE_ROUTE_LAUNCH_AS(TT, V, false)
+  if (scored) MOE_ROUTE_LAUNCH_AS(TT, V, true); else MOE_ROUTE_LAUNCH_AS(TT, V, false)
 #define MOE_ROUTE_LAUNCH_AS(TT, V, SQ)                                                          \
   hipLaunchKernelGGL((moe_route_kernel<TT, V, SQ>), dim3(T), dim3(MOE_THREADS), lds, stream,      \
-                     (const TT*)x, ldx, router, bias, T, D, E, top, sq, idx, wts)
+                     (const TT*)x, ldx, router, bias, T, D, E, top, sq, gates, idx, wts)
   if (x_is_bf16) {
     if (vec) { MOE_ROUTE_LAUNCH(bf16_t, 4); } else { MOE_ROUTE_LAUNCH(bf16_t, 1); }
   } else {
@@ -198,37 +214,40 @@ static int moe_route_launch(const void* x, int ldx, int x_is_bf16, const float* 
 }
 
 extern "C" int kappai_moe_route(const void* x, int ldx, int x_is_bf16, const float* router,
-                                const float* bias, int T, int D, int E, int top, int* idx,
-                                float* wts, hipStream_t stream) {
+                                const float* bias, int T, int D, int E, int top, float* gates,
+                                int* idx, float* wts, hipStream_t stream) {
   return moe_route_launch(x, ldx, x_is_bf16, router, bias, T, D, E, top, false,
-                          moe_squashed_choice{nullptr, 1, 1, 1.0f}, idx, wts, stream);
+                          moe_scored_choice{nullptr, 1, 1, 0, 1, 1.0f}, gates, idx, wts, stream);
 }
 
-extern "C" int kappai_moe_route_squashed(const void* x, int ldx, int x_is_bf16,
-                                         const float* router, const float* bias,
-                                         const float* correction, int groups, int keep,
-                                         float scale, int T, int D, int E, int top, int* idx,
-                                         float* wts, hipStream_t stream) {
+extern "C" int kappai_moe_route_scored(const void* x, int ldx, int x_is_bf16, const float* router,
+                                       const float* bias, const float* correction, int groups,
+                                       int keep, int over_all, int best, float scale, int T,
+                                       int D, int E, int top, float* gates, int* idx, float* wts,
+                                       hipStream_t stream) {
   return moe_route_launch(x, ldx, x_is_bf16, router, bias, T, D, E, top, true,
-                          moe_squashed_choice{correction, groups, keep, scale}, idx, wts, stream);
+                          moe_scored_choice{correction, groups, keep, over_all, best, scale},
+                          gates, idx, wts, stream);
 }
 
 // The pairs sorted by expert, stably and without atomics.  The waves of one block each take a
 // run of the pairs, 64 at a time: a lane finds the lanes with its own expert by one ballot a bit of
 // the expert's number and its place among them by counting those below.  Pass 1 counts per wave
 // and expert; then every expert's run gets its first slot (a multiple of MOE_TILE_M) and every
-// wave its place in the run; pass 2 places.
+// wave its place in the run; pass 2 places.  A pair whose expert is none of the E (one that hands its input
+// on) gets slot -1.
 #define MOE_PLAN_MAX_WAVES 16
 
 __device__ __forceinline__ void moe_plan_pass(const int* __restrict__ idx, int p_lo, int p_hi,
-                                              int n_bits, int* cnt, const int* start, bool place,
+                                              int E, int n_bits, int* cnt, const int* start, bool place,
                                               int* __restrict__ slot_of_pair,
                                               int* __restrict__ pair_of_slot) {
   const int lane = threadIdx.x % WAVE;
   int next = p_lo + lane < p_hi ? idx[p_lo + lane] : 0;
   for (int p0 = p_lo; p0 < p_hi; p0 += WAVE) {
     const int p = p0 + lane, e = next;
-    const bool mine = p < p_hi;
+    const bool mine = p < p_hi && e < E;
+    if (place && p < p_hi && e >= E) slot_of_pair[p] = -1;
     next = p + WAVE < p_hi ? idx[p + WAVE] : 0;
     unsigned long long same = __ballot(mine);
     for (int b = 0; b < n_bits; ++b) {
@@ -270,7 +289,8 @@ __global__ __launch_bounds__(MOE_PLAN_MAX_WAVES * WAVE) void moe_plan_kernel(
   const int per = ((P + n_waves * WAVE - 1) / (n_waves * WAVE)) * WAVE;
   const int p_lo = min(P, wave * per), p_hi = min(P, p_lo + per);
   const int n_bits = E > 1 ? 32 - __clz(E - 1) : 0;
-  moe_plan_pass(idx, p_lo, p_hi, n_bits, cnt + wave * E, nullptr, false, slot_of_pair, pair_of_slot);
+  moe_plan_pass(idx, p_lo, p_hi, E, n_bits, cnt + wave * E, nullptr, false, slot_of_pair,
+                pair_of_slot);
   __syncthreads();
   // the runs' lengths and, inside a run, the waves one after the other
   for (int e = tid; e < E; e += nt) {
@@ -299,7 +319,7 @@ __global__ __launch_bounds__(MOE_PLAN_MAX_WAVES * WAVE) void moe_plan_kernel(
     for (int i = 0; i < n; ++i) tile_expert[first / MOE_TILE_M + i] = e;
   }
   __syncthreads();
-  moe_plan_pass(idx, p_lo, p_hi, n_bits, cnt + wave * E, start + wave * E, true, slot_of_pair,
+  moe_plan_pass(idx, p_lo, p_hi, E, n_bits, cnt + wave * E, start + wave * E, true, slot_of_pair,
                 pair_of_slot);
 }
 
@@ -321,22 +341,38 @@ extern "C" int kappai_moe_plan(const int* idx, int P, int E, int n_tiles, int* s
 __device__ __forceinline__ float silu_exact(float g) { return g / (1.0f + expf(-g)); }
 __device__ __forceinline__ float relu_squared(float z) { const float r = fmaxf(z, 0.f); return r * r; }
 
+// The clamped gate: g = min(g, limit), u = clamp(u, -limit, limit), g sigmoid(slope g) (u + shift).
+struct moe_clamp { float limit, slope, shift; };
+__device__ __forceinline__ float clamped_gate(float g, float u, const moe_clamp& c) {
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit);
+  return g / (1.0f + expf(-c.slope * g)) * (u + c.shift);
+}
+
+// The forms of the experts' products: 0 the slots' own rows, one matrix, float results; 1 gathered
+// rows, two matrices, silu(g) u; 2 gathered rows, one matrix, relu(z)^2; 3 as 1 with the clamped gate.
+constexpr bool moe_two(int form) { return form == 1 || form == 3; }
+template <int FORM>
+__device__ __forceinline__ float moe_gated(float g, float u, const moe_clamp& c) {
+  return FORM == 3 ? clamped_gate(g, u, c) : silu_exact(g) * u;
+}
+
 // Half a tile (MOE_HALF_M slots) of one expert times MOE_TILE_N rows of its matrix, float sums on
 // the vector units (this is the 32-bit path, and the path of any shape).  GATED: the rows are
-// gathered from x by pair / top, two matrices, out = silu(g) * u in T; GATED == 2: gathered rows,
-// one matrix, out = relu(x W^T)^2 in T; else the rows are the slots of `a` themselves and out is
-// float.
+// gathered from x by pair / top, two matrices, out = gate(g, u) in T (forms 1 and 3); GATED == 2:
+// gathered rows, one matrix, out = relu(x W^T)^2 in T; else the rows are the slots of `a`
+// themselves and out is float.
 template <typename T, int GATED>
 __global__ __launch_bounds__(MOE_THREADS) void moe_gemm_kernel(
     const T* __restrict__ a, int lda, const T* __restrict__ w0, const T* __restrict__ w1, int N,
     int K, const int* __restrict__ tile_expert, const int* __restrict__ pair_of_slot, int top,
-    void* __restrict__ out_v) {
+    moe_clamp clamp, void* __restrict__ out_v) {
   const int tile = blockIdx.x / 2, slot0 = blockIdx.x * MOE_HALF_M;
   const int e = tile_expert[tile];
   if (e < 0) return;
   __shared__ float As[MOE_TILE_K][MOE_HALF_M + 1];
   __shared__ float W0s[MOE_TILE_K][MOE_TILE_N + 1];
-  __shared__ float W1s[GATED == 1 ? MOE_TILE_K : 1][MOE_TILE_N + 1];
+  __shared__ float W1s[moe_two(GATED) ? MOE_TILE_K : 1][MOE_TILE_N + 1];
   __shared__ int src_row[MOE_HALF_M];
   const int tid = threadIdx.x;
   if (tid < MOE_HALF_M) {
@@ -347,7 +383,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_gemm_kernel(
   __syncthreads();
   const int n0 = blockIdx.y * MOE_TILE_N;
   const T* W0 = w0 + (size_t)e * N * K;
-  const T* W1 = GATED == 1 ? w1 + (size_t)e * N * K : nullptr;
+  const T* W1 = moe_two(GATED) ? w1 + (size_t)e * N * K : nullptr;
   const int ty = tid / 16, tx = tid % 16;
   float acc0[2][4] = {}, acc1[2][4] = {};
   const int am = tid / 8, ak = (tid % 8) * 4;       // this thread's piece of the A tile
@@ -364,7 +400,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_gemm_kernel(
       const int k = k0 + wk + i, n = n0 + wn;
       const bool ok = n < N && k < K;
       W0s[wk + i][wn] = ok ? to_f32(W0[(size_t)n * K + k]) : 0.f;
-      if (GATED == 1) W1s[wk + i][wn] = ok ? to_f32(W1[(size_t)n * K + k]) : 0.f;
+      if (moe_two(GATED)) W1s[wk + i][wn] = ok ? to_f32(W1[(size_t)n * K + k]) : 0.f;
     }
     __syncthreads();
 #pragma unroll 8
@@ -375,7 +411,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_gemm_kernel(
         const float b0 = W0s[k][tx + 16 * j];
         acc0[0][j] = fmaf(a0, b0, acc0[0][j]);
         acc0[1][j] = fmaf(a1, b0, acc0[1][j]);
-        if (GATED == 1) {
+        if (moe_two(GATED)) {
           const float b1 = W1s[k][tx + 16 * j];
           acc1[0][j] = fmaf(a0, b1, acc1[0][j]);
           acc1[1][j] = fmaf(a1, b1, acc1[1][j]);
@@ -393,8 +429,8 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_gemm_kernel(
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx + 16 * j;
       if (n >= N) continue;
-      if (GATED == 1)
-        from_f32((T*)out_v + slot * N + n, silu_exact(acc0[i][j]) * acc1[i][j]);
+      if (moe_two(GATED))
+        from_f32((T*)out_v + slot * N + n, moe_gated<GATED>(acc0[i][j], acc1[i][j], clamp));
       else if (GATED == 2)
         from_f32((T*)out_v + slot * N + n, relu_squared(acc0[i][j]));
       else
@@ -405,21 +441,22 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_gemm_kernel(
 
 extern "C" int kappai_moe_gemm(const void* a, int lda, const void* w0, const void* w1, int N,
                                int K, const int* tile_expert, const int* pair_of_slot, int top,
-                               int n_tiles, void* out, int gated, int is_bf16,
-                               hipStream_t stream) {
+                               int n_tiles, void* out, int gated, float limit, float slope,
+                               float shift, int is_bf16, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   const dim3 grid(n_tiles * (MOE_TILE_M / MOE_HALF_M), (N + MOE_TILE_N - 1) / MOE_TILE_N);
   if (grid.y > 65535) return (int)hipErrorInvalidValue;
 #define MOE_GEMM_LAUNCH(TT, G)                                                                  \
   hipLaunchKernelGGL((moe_gemm_kernel<TT, G>), grid, dim3(MOE_THREADS), 0, stream, (const TT*)a, \
-                     lda, (const TT*)w0, (const TT*)w1, N, K, tile_expert, pair_of_slot, top, out)
-  if (gated < 0 || gated > 2) return (int)hipErrorInvalidValue;
+                     lda, (const TT*)w0, (const TT*)w1, N, K, tile_expert, pair_of_slot, top, clamp, out)
+  if (gated < 0 || gated > 3) return (int)hipErrorInvalidValue;
+  const moe_clamp clamp{limit, slope, shift};
   if (is_bf16) {
     if (gated == 1) MOE_GEMM_LAUNCH(bf16_t, 1); else if (gated == 2) MOE_GEMM_LAUNCH(bf16_t, 2);
-    else MOE_GEMM_LAUNCH(bf16_t, 0);
+    else if (gated == 3) MOE_GEMM_LAUNCH(bf16_t, 3); else MOE_GEMM_LAUNCH(bf16_t, 0);
   } else {
     if (gated == 1) MOE_GEMM_LAUNCH(float, 1); else if (gated == 2) MOE_GEMM_LAUNCH(float, 2);
-    else MOE_GEMM_LAUNCH(float, 0);
+    else if (gated == 3) MOE_GEMM_LAUNCH(float, 3); else MOE_GEMM_LAUNCH(float, 0);
   }
 #undef MOE_GEMM_LAUNCH
   KAPPAI_RETURN_LAUNCH_STATUS();
@@ -451,9 +488,10 @@ template <int GATED, int NT, int U, bool WF, bool BYROW>
 __global__ __launch_bounds__(MOE_MFMA_WAVES * WAVE) void moe_gemm_mfma_kernel(
     const bf16_t* __restrict__ a, int lda, const bf16_t* __restrict__ w0,
     const bf16_t* __restrict__ w1, int N, int K, const int* __restrict__ tile_expert,
-    const int* __restrict__ pair_of_slot, int top, int n_tiles, void* __restrict__ out_v) {
+    const int* __restrict__ pair_of_slot, int top, int n_tiles, moe_clamp clamp,
+    void* __restrict__ out_v) {
   constexpr int MT = MOE_TILE_M / 16;
-  constexpr int NG = GATED == 1 ? 2 : 1;
+  constexpr int NG = moe_two(GATED) ? 2 : 1;
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
   const int tile = BYROW ? blockIdx.x * MOE_MFMA_WAVES + wave : blockIdx.x;
   if (tile >= n_tiles) return;
@@ -482,7 +520,7 @@ __global__ __launch_bounds__(MOE_MFMA_WAVES * WAVE) void moe_gemm_mfma_kernel(
                                lane * 8
                          : ((size_t)e * N + (w_ok[j] ? n : 0)) * K + kg;
     wrow[0][j] = w0 + at;
-    if (GATED == 1) wrow[1][j] = w1 + at;
+    if (moe_two(GATED)) wrow[1][j] = w1 + at;
   }
   moe_f32x4_t acc[NG][NT][MT];
 #pragma unroll
@@ -544,9 +582,9 @@ __global__ __launch_bounds__(MOE_MFMA_WAVES * WAVE) void moe_gemm_mfma_kernel(
       for (int j = 0; j < NT; ++j) {
         const int n = n0 + 16 * j + col;
         if (n >= N) continue;
-        if (GATED == 1)
+        if (moe_two(GATED))
           ((bf16_t*)out_v)[slot * N + n] =
-              f32_to_bf16(silu_exact(acc[0][j][t][v]) * acc[GATED == 1 ? 1 : 0][j][t][v]);
+              f32_to_bf16(moe_gated<GATED>(acc[0][j][t][v], acc[NG - 1][j][t][v], clamp));
         else if (GATED == 2)
           ((bf16_t*)out_v)[slot * N + n] = f32_to_bf16(relu_squared(acc[0][j][t][v]));
         else
@@ -559,7 +597,8 @@ __global__ __launch_bounds__(MOE_MFMA_WAVES * WAVE) void moe_gemm_mfma_kernel(
 // the experts' matrices: one column tile a wave (twice the blocks) and two steps of K a load.
 extern "C" int kappai_moe_gemm_mfma(const void* a, int lda, const void* w0, const void* w1, int N,
                                     int K, const int* tile_expert, const int* pair_of_slot,
-                                    int top, int n_tiles, void* out, int gated, int few,
+                                    int top, int n_tiles, void* out, int gated, float limit,
+                                    float slope, float shift, int few,
                                     int w_frag, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   if ((K % 8) || (lda % 8) || ((uintptr_t)a % 16) || ((uintptr_t)w0 % 16) || ((uintptr_t)w1 % 16))
@@ -574,12 +613,15 @@ extern "C" int kappai_moe_gemm_mfma(const void* a, int lda, const void* w0, cons
       BR_ ? dim3((n_tiles + MOE_MFMA_WAVES - 1) / MOE_MFMA_WAVES, (N + 16 * NT_ - 1) / (16 * NT_)) \
           : dim3(n_tiles, (N + 16 * NT_ * MOE_MFMA_WAVES - 1) / (16 * NT_ * MOE_MFMA_WAVES)),      \
       block, 0, stream, (const bf16_t*)a, lda, (const bf16_t*)w0, (const bf16_t*)w1, N, K,         \
-      tile_expert, pair_of_slot, top, n_tiles, out)
-  if (gated < 0 || gated > 2) return (int)hipErrorInvalidValue;
+      tile_expert, pair_of_slot, top, n_tiles, clamp, out)
+  if (gated < 0 || gated > 3) return (int)hipErrorInvalidValue;
+  const moe_clamp clamp{limit, slope, shift};
   if (gated == 1) {
     if (few) { MOE_MFMA_LAUNCH(1, 1, 2, false); } else { MOE_MFMA_LAUNCH(1, 4, 1, true); }
   } else if (gated == 2) {
     if (few) { MOE_MFMA_LAUNCH(2, 2, 2, false); } else { MOE_MFMA_LAUNCH(2, 4, 1, true); }
+  } else if (gated == 3) {
+    if (few) { MOE_MFMA_LAUNCH(3, 1, 2, false); } else { MOE_MFMA_LAUNCH(3, 4, 1, true); }
   } else {
     if (few) { MOE_MFMA_LAUNCH(0, 2, 2, false); } else { MOE_MFMA_LAUNCH(0, 4, 1, true); }
   }
@@ -588,10 +630,13 @@ extern "C" int kappai_moe_gemm_mfma(const void* a, int lda, const void* w0, cons
   KAPPAI_RETURN_LAUNCH_STATUS();
 }
 
+// `also`: what every row gets beside its experts (times also_gate[t] where there is a gate); `x`
+// [T, D]: the rows themselves, for pairs of slot -1 (experts that hand their input on).
 __global__ __launch_bounds__(MOE_THREADS) void moe_combine_kernel(
     const float* __restrict__ y, const int* __restrict__ slot_of_pair,
     const float* __restrict__ wts, int top, int D, const void* __restrict__ also,
-    int also_is_bf16, int also_parts, size_t also_plane, float* __restrict__ out) {
+    int also_is_bf16, int also_parts, size_t also_plane, const float* __restrict__ also_gate,
+    const void* __restrict__ x, int ldx, int x_is_bf16, float* __restrict__ out) {
   const int t = blockIdx.x;
   for (int n = blockIdx.y * MOE_THREADS + threadIdx.x; n < D; n += gridDim.y * MOE_THREADS) {
     // what every row gets beside its experts (a shared expert's result: rows, or float planes
@@ -602,22 +647,31 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_combine_kernel(
       if (also_is_bf16) acc = bf16_to_f32(((const bf16_t*)also)[at]);
       else
         for (int p = 0; p < also_parts; ++p) acc += ((const float*)also)[p * also_plane + at];
+      if (also_gate != nullptr) acc *= also_gate[t];
     }
-    for (int k = 0; k < top; ++k)
-      acc = fmaf(wts[(size_t)t * top + k], y[(size_t)slot_of_pair[(size_t)t * top + k] * D + n],
-                 acc);
+    for (int k = 0; k < top; ++k) {
+      const int slot = slot_of_pair[(size_t)t * top + k];
+      float v = 0.f;
+      if (slot >= 0) v = y[(size_t)slot * D + n];
+      else if (x != nullptr)
+        v = x_is_bf16 ? bf16_to_f32(((const bf16_t*)x)[(size_t)t * ldx + n])
+                      : ((const float*)x)[(size_t)t * ldx + n];
+      acc = fmaf(wts[(size_t)t * top + k], v, acc);
+    }
     out[(size_t)t * D + n] = acc;
   }
 }
 
 extern "C" int kappai_moe_combine(const float* y, const int* slot_of_pair, const float* wts, int T,
                                   int top, int D, const void* also, int also_is_bf16,
-                                  int also_parts, float* out, hipStream_t stream) {
+                                  int also_parts, const float* also_gate, const void* x, int ldx,
+                                  int x_is_bf16, float* out, hipStream_t stream) {
   if (T <= 0) return 0;
   if (also && also_parts < 1) return (int)hipErrorInvalidValue;
   // few rows: a thread a column, so that all its loads are asked for at once
   const int col_blocks = T <= 512 ? min(64, (D + MOE_THREADS - 1) / MOE_THREADS) : 1;
-  hipLaunchKernelGGL(moe_combine_kernel, dim3(T, col_blocks), dim3(MOE_THREADS), 0, stream, y, slot_of_pair,
-                     wts, top, D, also, also_is_bf16, also_parts, (size_t)T * D, out);
+  hipLaunchKernelGGL(moe_combine_kernel, dim3(T, col_blocks), dim3(MOE_THREADS), 0, stream, y,
+                     slot_of_pair, wts, top, D, also, also_is_bf16, also_parts, (size_t)T * D,
+                     also_gate, x, ldx, x_is_bf16, out);
   KAPPAI_RETURN_LAUNCH_STATUS();
 }

@@ -1380,17 +1380,38 @@ def scale_add_positions(x: torch.Tensor, scale: float, table: torch.Tensor,
 GLU_SILU, GLU_GELU_TANH = 0, 1
 
 
-def glu(gate_up: torch.Tensor, kind: int) -> torch.Tensor:
+GLU_CLAMPED = 2
+
+
+@dataclass(frozen=True)
+class ClampedGate:
+    """The gate ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``, ``g sigmoid(slope g) (u +
+    shift)``."""
+    limit: float
+    slope: float = 1.702
+    shift: float = 1.0
+
+    def c_args(self):
+        return _c_float(self.limit), _c_float(self.slope), _c_float(self.shift)
+
+
+_NO_CLAMP = (_c_float(0.0), _c_float(0.0), _c_float(0.0))
+
+
+def glu(gate_up: torch.Tensor, kind: int, clamp: Optional[ClampedGate] = None) -> torch.Tensor:
     """``act(gate_up[:, :F]) * gate_up[:, F:]`` for a fused [T, 2F] projection; ``kind``:
-    ``GLU_SILU`` or ``GLU_GELU_TANH`` (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))))."""
+    ``GLU_SILU``, ``GLU_GELU_TANH`` (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))) or
+    ``GLU_CLAMPED`` (``clamp``: its constants)."""
     _gpu("gate_up", gate_up, (F32, BF16))
     _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, "glu: [T, 2F] is needed")
-    _need(kind in (GLU_SILU, GLU_GELU_TANH), lambda: f"glu: unknown activation {kind}")
+    _need(kind in (GLU_SILU, GLU_GELU_TANH, GLU_CLAMPED),
+          lambda: f"glu: unknown activation {kind}")
+    _need((kind == GLU_CLAMPED) == (clamp is not None), "glu: the clamped gate and its constants")
     T, F = gate_up.shape[0], gate_up.shape[1] // 2
     out = torch.empty((T, F), dtype=gate_up.dtype, device=gate_up.device)
     check(library("elementwise").kappai_glu(
         _ptr(gate_up), _ptr(out), _c_int(T), _c_int(F), _c_int(_is_bf16(gate_up.dtype)),
-        _c_int(kind), _stream()), "glu")
+        _c_int(kind), *(clamp.c_args() if clamp else _NO_CLAMP), _stream()), "glu")
     return out
 
 
@@ -1597,64 +1618,75 @@ def diff_combine(ctx: torch.Tensor, n_heads: int, n_kv_heads: int, vdim: int, he
 MOE_MAX_TOP = 16
 
 
+def _moe_router(what, x, router, top, bias, gate):
+    """Checks of both routers; returns (T, D, experts, gates or None)."""
+    _gpu("x", x, (F32, BF16), contiguous=False)
+    _gpu("router", router, F32)
+    T, D = x.shape
+    E = router.shape[0] - (1 if gate else 0)
+    if bias is not None:
+        _gpu("bias", bias, F32)
+        _need(bias.shape == (E,), lambda: f"{what}: bias {tuple(bias.shape)}")
+    _need(router.dim() == 2 and router.shape[1] == D and x.stride(1) == 1
+          and 1 <= top <= min(E, MOE_MAX_TOP),
+          lambda: f"{what}: x {tuple(x.shape)}, router {tuple(router.shape)}, top {top}")
+    return T, D, E, torch.empty((T,), dtype=F32, device=x.device) if gate else None
+
+
 def moe_route(x: torch.Tensor, router: torch.Tensor, top: int,
               bias: Optional[torch.Tensor] = None):
     """Router logits ``x router^T (+ bias)`` in float32, the ``top`` largest of a row chosen (the
     lowest index wins a tie), weights = softmax over the chosen logits.  Returns (experts [T, top]
     int32, weights [T, top] float32), the largest first."""
-    _gpu("x", x, (F32, BF16), contiguous=False)
-    _gpu("router", router, F32)
-    if bias is not None:
-        _gpu("bias", bias, F32)
-        _need(bias.shape == (router.shape[0],), lambda: f"moe_route: bias {tuple(bias.shape)}")
-    T, D = x.shape
-    E = router.shape[0]
-    _need(router.shape == (E, D) and x.stride(1) == 1 and 1 <= top <= min(E, MOE_MAX_TOP),
-          lambda: f"moe_route: x {tuple(x.shape)}, router {tuple(router.shape)}, top {top}")
+    T, D, E, _ = _moe_router("moe_route", x, router, top, bias, False)
     idx = torch.empty((T, top), dtype=I32, device=x.device)
     wts = torch.empty((T, top), dtype=F32, device=x.device)
     check(library("moe").kappai_moe_route(
         _ptr(x), _c_int(x.stride(0)), _c_int(_is_bf16(x.dtype)), _ptr(router), _ptr(bias),
-        _c_int(T), _c_int(D), _c_int(E), _c_int(top), _ptr(idx), _ptr(wts), _stream()),
+        _c_int(T), _c_int(D), _c_int(E), _c_int(top), _vp(0), _ptr(idx), _ptr(wts), _stream()),
         "moe_route")
     return idx, wts
 
 
-def moe_route_squashed(x: torch.Tensor, router: torch.Tensor, top: int, scale: float = 1.0,
-                       correction: Optional[torch.Tensor] = None, groups: int = 1,
-                       keep_groups: int = 1, bias: Optional[torch.Tensor] = None):
-    """Router logits ``z = x router^T (+ bias)`` in float32, every logit squashed by itself: score
-    ``s = sigmoid(z)``.  Chosen are the ``top`` experts with the largest ``s + correction``
-    (correction [E] float32 or None; the lowest index wins a tie) among the ``keep_groups`` best of
-    ``groups`` equal groups of neighbouring experts, a group's worth being the sum of its two
-    largest such values.  The weights are ``s * scale`` of the chosen ones.  Returns (experts [T,
-    top] int32, weights [T, top] float32), in the order of the choice."""
-    _gpu("x", x, (F32, BF16), contiguous=False)
-    _gpu("router", router, F32)
-    T, D = x.shape
-    E = router.shape[0]
-    for name, t in (("bias", bias), ("correction", correction)):
-        if t is not None:
-            _gpu(name, t, F32)
-            _need(t.shape == (E,), lambda: f"moe_route_squashed: {name} {tuple(t.shape)}")
-    _need(router.shape == (E, D) and x.stride(1) == 1 and 1 <= top <= MOE_MAX_TOP,
-          lambda: f"moe_route_squashed: x {tuple(x.shape)}, router {tuple(router.shape)}, top {top}")
+SCORE_KINDS = {"sigmoid": 0, "softmax": 1}
+
+
+def moe_route_scored(x: torch.Tensor, router: torch.Tensor, top: int, scale: float = 1.0,
+                     correction: Optional[torch.Tensor] = None, groups: int = 1,
+                     keep_groups: int = 1, bias: Optional[torch.Tensor] = None,
+                     score: str = "sigmoid", group_best: int = 2, gate: bool = False):
+    """Router logits ``z = x router^T (+ bias)`` in float32 and a score an expert: ``s =
+    sigmoid(z)`` of its own logit, or (``score`` "softmax") ``s = softmax(z)`` over all experts.
+    Chosen are the ``top`` experts with the largest ``s + correction`` (correction [E] float32 or
+    None; the lowest index wins a tie) among the ``keep_groups`` best of ``groups`` equal groups of
+    neighbouring experts, a group's worth being the sum of its ``group_best`` (1 or 2) largest such
+    values.  The weights are ``s * scale`` of the chosen ones.  Returns (experts [T, top] int32,
+    weights [T, top] float32), in the order of the choice.  ``gate``: the router's last row is no
+    expert's; sigmoid of its logit, [T] float32, is returned as a third result."""
+    T, D, E, gates = _moe_router("moe_route_scored", x, router, top, bias, gate)
+    if correction is not None:
+        _gpu("correction", correction, F32)
+        _need(correction.shape == (E,),
+              lambda: f"moe_route_scored: correction {tuple(correction.shape)}")
     _need(groups >= 1 and E % groups == 0 and 1 <= keep_groups <= groups
-          and top <= E // groups * keep_groups,
-          lambda: f"moe_route_squashed: {top} of {E} experts, {keep_groups} of {groups} groups")
+          and top <= E // groups * keep_groups and score in SCORE_KINDS and group_best in (1, 2),
+          lambda: f"moe_route_scored: {top} of {E} experts, {keep_groups} of {groups} groups, "
+                  f"score {score!r}, {group_best} values a group")
     idx = torch.empty((T, top), dtype=I32, device=x.device)
     wts = torch.empty((T, top), dtype=F32, device=x.device)
-    check(library("moe").kappai_moe_route_squashed(
+    check(library("moe").kappai_moe_route_scored(
         _ptr(x), _c_int(x.stride(0)), _c_int(_is_bf16(x.dtype)), _ptr(router), _ptr(bias),
-        _ptr(correction), _c_int(groups), _c_int(keep_groups), _c_float(scale), _c_int(T),
-        _c_int(D), _c_int(E), _c_int(top), _ptr(idx), _ptr(wts), _stream()), "moe_route_squashed")
-    return idx, wts
+        _ptr(correction), _c_int(groups), _c_int(keep_groups), _c_int(SCORE_KINDS[score]),
+        _c_int(group_best), _c_float(scale), _c_int(T), _c_int(D), _c_int(E), _c_int(top),
+        _ptr(gates), _ptr(idx), _ptr(wts), _stream()), "moe_route_scored")
+    return (idx, wts, gates) if gate else (idx, wts)
 
 
 @dataclass
 class MoePlan:
-    """The step's (row, choice) pairs in expert order: ``slot_of_pair`` [T top], ``pair_of_slot``
-    [tiles * tile_rows] (-1: empty), ``tile_expert`` [tiles] (-1: unused)."""
+    """The step's (row, choice) pairs in expert order: ``slot_of_pair`` [T top] (-1: the pair's
+    expert hands its input on), ``pair_of_slot`` [tiles * tile_rows] (-1: empty), ``tile_expert``
+    [tiles] (-1: unused)."""
     slot_of_pair: torch.Tensor
     pair_of_slot: torch.Tensor
     tile_expert: torch.Tensor
@@ -1664,6 +1696,8 @@ class MoePlan:
 
 
 def moe_plan(experts: torch.Tensor, n_experts: int) -> MoePlan:
+    """``experts`` [T, top]; numbers from ``n_experts`` on are experts without matrices, whose pairs
+    get no place."""
     _gpu("experts", experts, I32)
     T, top = experts.shape
     P = T * top
@@ -1727,9 +1761,10 @@ def _moe_on_matrix_cores(a: torch.Tensor, lda: int, K: int, *matrices) -> bool:
 
 
 def moe_experts_gated(x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor,
-                      plan: MoePlan) -> torch.Tensor:
-    """``silu(x Wg[e]^T) * (x Wu[e]^T)`` for every slot of the plan ([slots, F], the dtype of
-    ``x``; empty slots are left unwritten).  ``w_gate``, ``w_up``: [E, F, D]."""
+                      plan: MoePlan, clamp: Optional[ClampedGate] = None) -> torch.Tensor:
+    """``silu(x Wg[e]^T) * (x Wu[e]^T)`` (``clamp``: the clamped gate in place of silu) for every
+    slot of the plan ([slots, F], the dtype of ``x``; empty slots are left unwritten).  ``w_gate``,
+    ``w_up``: [E, F, D]."""
     _gpu("x", x, (F32, BF16), contiguous=False)
     E, F, D = w_gate.shape
     (w_gate, frag), (w_up, frag_up) = _moe_matrix(w_gate), _moe_matrix(w_up)
@@ -1740,19 +1775,21 @@ def moe_experts_gated(x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor,
           lambda: f"moe_experts_gated: x {tuple(x.shape)}, matrices {(E, F, D)}")
     out = torch.empty((plan.n_tiles * plan.tile_rows, F), dtype=x.dtype, device=x.device)
     mfma = _moe_on_matrix_cores(x, x.stride(0), D, w_gate, w_up)
+    form, consts = (3, clamp.c_args()) if clamp else (1, _NO_CLAMP)
     _need(mfma or not frag, "moe_experts_gated: matrices in fragment order need bfloat16 rows "
           "with 16-byte aligned starts")
     if mfma:
         check(library("moe").kappai_moe_gemm_mfma(
             _ptr(x), _c_int(x.stride(0)), _ptr(w_gate), _ptr(w_up), _c_int(F), _c_int(D),
             _ptr(plan.tile_expert), _ptr(plan.pair_of_slot), _c_int(plan.top),
-            _c_int(plan.n_tiles), _ptr(out), _c_int(1), _c_int(_moe_few(plan)), _c_int(frag),
-            _stream()), "moe_gemm_mfma (gate, up)")
+            _c_int(plan.n_tiles), _ptr(out), _c_int(form), *consts, _c_int(_moe_few(plan)),
+            _c_int(frag), _stream()), "moe_gemm_mfma (gate, up)")
         return out
     check(library("moe").kappai_moe_gemm(
         _ptr(x), _c_int(x.stride(0)), _ptr(w_gate), _ptr(w_up), _c_int(F), _c_int(D),
         _ptr(plan.tile_expert), _ptr(plan.pair_of_slot), _c_int(plan.top), _c_int(plan.n_tiles),
-        _ptr(out), _c_int(1), _c_int(_is_bf16(x.dtype)), _stream()), "moe_gemm (gate, up)")
+        _ptr(out), _c_int(form), *consts, _c_int(_is_bf16(x.dtype)), _stream()),
+        "moe_gemm (gate, up)")
     return out
 
 
@@ -1773,13 +1810,13 @@ def moe_experts_activated(x: torch.Tensor, w_up: torch.Tensor, plan: MoePlan) ->
         check(library("moe").kappai_moe_gemm_mfma(
             _ptr(x), _c_int(x.stride(0)), _ptr(w_up), _vp(0), _c_int(F), _c_int(D),
             _ptr(plan.tile_expert), _ptr(plan.pair_of_slot), _c_int(plan.top),
-            _c_int(plan.n_tiles), _ptr(out), _c_int(2), _c_int(_moe_few(plan)), _c_int(frag),
-            _stream()), "moe_gemm_mfma (up, squared relu)")
+            _c_int(plan.n_tiles), _ptr(out), _c_int(2), *_NO_CLAMP, _c_int(_moe_few(plan)),
+            _c_int(frag), _stream()), "moe_gemm_mfma (up, squared relu)")
         return out
     check(library("moe").kappai_moe_gemm(
         _ptr(x), _c_int(x.stride(0)), _ptr(w_up), _vp(0), _c_int(F), _c_int(D),
         _ptr(plan.tile_expert), _ptr(plan.pair_of_slot), _c_int(plan.top), _c_int(plan.n_tiles),
-        _ptr(out), _c_int(2), _c_int(_is_bf16(x.dtype)), _stream()),
+        _ptr(out), _c_int(2), *_NO_CLAMP, _c_int(_is_bf16(x.dtype)), _stream()),
         "moe_gemm (up, squared relu)")
     return out
 
@@ -1799,52 +1836,131 @@ def moe_experts_down(act: torch.Tensor, w_down: torch.Tensor, plan: MoePlan) -> 
         check(library("moe").kappai_moe_gemm_mfma(
             _ptr(act), _c_int(F), _ptr(w_down), _vp(0), _c_int(D), _c_int(F),
             _ptr(plan.tile_expert), _ptr(plan.pair_of_slot), _c_int(plan.top),
-            _c_int(plan.n_tiles), _ptr(out), _c_int(0), _c_int(_moe_few(plan)), _c_int(frag),
-            _stream()), "moe_gemm_mfma (down)")
+            _c_int(plan.n_tiles), _ptr(out), _c_int(0), *_NO_CLAMP, _c_int(_moe_few(plan)),
+            _c_int(frag), _stream()), "moe_gemm_mfma (down)")
         return out
     check(library("moe").kappai_moe_gemm(
         _ptr(act), _c_int(F), _ptr(w_down), _vp(0), _c_int(D), _c_int(F),
         _ptr(plan.tile_expert), _ptr(plan.pair_of_slot), _c_int(plan.top), _c_int(plan.n_tiles),
-        _ptr(out), _c_int(0), _c_int(_is_bf16(act.dtype)), _stream()), "moe_gemm (down)")
+        _ptr(out), _c_int(0), *_NO_CLAMP, _c_int(_is_bf16(act.dtype)), _stream()),
+        "moe_gemm (down)")
     return out
 
 
+def _also_parts(what, also, T, D):
+    """Checks ``also`` ([T, D] or float32 planes [S, T, D]); returns (bfloat16?, planes)."""
+    _gpu("also", also, (F32, BF16))
+    _need(also.dim() == 2 or (also.dim() == 3 and also.dtype == F32)
+          and tuple(also.shape[-2:]) == (T, D), lambda: f"{what}: also {tuple(also.shape)}")
+    _need(tuple(also.shape[-2:]) == (T, D), lambda: f"{what}: also {tuple(also.shape)}")
+    return _is_bf16(also.dtype), also.shape[0] if also.dim() == 3 else 1
+
+
+def _terms_args(what, T, D, also, also_gate, rows):
+    """What stands beside the chosen experts' results, as the kernels take it."""
+    isb, parts = _also_parts(what, also, T, D) if also is not None else (0, 1)
+    if also_gate is not None:
+        _gpu("also_gate", also_gate, F32)
+        _need(also is not None and also_gate.shape == (T,),
+              lambda: f"{what}: also_gate {tuple(also_gate.shape)}")
+    if rows is not None:
+        _gpu("rows", rows, (F32, BF16), contiguous=False)
+        _need(tuple(rows.shape) == (T, D) and rows.stride(1) == 1,
+              lambda: f"{what}: rows {tuple(rows.shape)}")
+    return (_ptr(also), _c_int(isb), _c_int(parts), _ptr(also_gate), _ptr(rows),
+            _c_int(rows.stride(0) if rows is not None else 0),
+            _c_int(_is_bf16(rows.dtype) if rows is not None else 0))
+
+
 def moe_combine(y: torch.Tensor, weights: torch.Tensor, plan: MoePlan,
-                also: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``out[t] = (also[t] +) sum_k weights[t, k] * y[slot of (t, k)]`` in the order of k: float32
-    [T, D].  ``also``: what every row gets beside its experts, [T, D] in float32 or bfloat16, or
-    float32 partial sums [S, T, D] (added in order)."""
+                also: Optional[torch.Tensor] = None, also_gate: Optional[torch.Tensor] = None,
+                rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out[t] = (also[t] (* also_gate[t]) +) sum_k weights[t, k] * y[slot of (t, k)]`` in the
+    order of k: float32 [T, D].  ``also``: what every row gets beside its experts, [T, D] in float32
+    or bfloat16, or float32 partial sums [S, T, D] (added in order); ``also_gate`` [T] float32.
+    ``rows`` [T, D]: the mixture's input, for experts that hand it on (slot -1)."""
     _gpu("y", y, F32)
     _gpu("weights", weights, F32)
     T, top = weights.shape
     D = y.shape[1]
     _need(top == plan.top and plan.slot_of_pair.shape[0] == T * top, "moe_combine: another plan")
-    parts = 1
-    if also is not None:
-        _gpu("also", also, (F32, BF16))
-        if also.dim() == 3:
-            _need(also.dtype == F32, "moe_combine: partial sums are float32")
-            parts = also.shape[0]
-        _need(tuple(also.shape[-2:]) == (T, D), lambda: f"moe_combine: also {tuple(also.shape)}")
     out = torch.empty((T, D), dtype=F32, device=y.device)
     check(library("moe").kappai_moe_combine(
         _ptr(y), _ptr(plan.slot_of_pair), _ptr(weights), _c_int(T), _c_int(top), _c_int(D),
-        _ptr(also), _c_int(_is_bf16(also.dtype) if also is not None else 0), _c_int(parts),
-        _ptr(out), _stream()), "moe_combine")
+        *_terms_args("moe_combine", T, D, also, also_gate, rows), _ptr(out), _stream()),
+        "moe_combine")
     return out
 
 
 @dataclass
 class ExpertTerms:
     """What a mixture's chosen experts left, not summed yet: ``y`` float32 [slots, D] in the plan's
-    order and ``weights`` [T, top].  The pass that reads it sums in the order of the choice
-    (``tanh_norm_step``), or ``combined()`` does."""
+    order and ``weights`` [T, top]; with what stands beside them (``also``, ``also_gate``, ``rows`` as
+    ``moe_combine`` takes them).  The pass that reads it sums in the order of the choice
+    (``tanh_norm_step``, ``rms_norm_step``), or ``combined()`` does."""
     y: torch.Tensor
     weights: torch.Tensor
     plan: MoePlan
+    also: Optional[torch.Tensor] = None
+    also_gate: Optional[torch.Tensor] = None
+    rows: Optional[torch.Tensor] = None
 
     def combined(self) -> torch.Tensor:
-        return moe_combine(self.y, self.weights, self.plan)
+        return moe_combine(self.y, self.weights, self.plan, also=self.also,
+                           also_gate=self.also_gate, rows=self.rows)
+
+
+RMS_STEP_MAX_WIDTH = 8192
+
+
+def rms_norm_step(resid: torch.Tensor, y=None, post=None, pre=None,
+                  rows: Optional[torch.Tensor] = None, rows_dtype=None) -> Optional[torch.Tensor]:
+    """RMS norms on both sides of a sublayer in one pass over the stream ``resid`` [T, D] float32:
+    ``resid += post(y)`` in place, and the rows ``pre(resid)`` in ``rows_dtype`` are returned.
+    ``post``, ``pre``: (weight [D] float32, eps) or None; ``y``: [T, D] in float32 or bfloat16,
+    float32 partial sums [S, T, D] (added in order first), ``ExpertTerms`` (summed first), or None;
+    ``post`` None: ``y`` is added as it is; ``pre`` None: no rows.  ``rows`` (int32): only these
+    rows are made, and the stream keeps its values.  Widths up to ``RMS_STEP_MAX_WIDTH``."""
+    _gpu("resid", resid, F32)
+    _need(resid.dim() == 2 and resid.shape[1] <= RMS_STEP_MAX_WIDTH,
+          lambda: f"rms_norm_step: resid {tuple(resid.shape)}")
+    T, D = resid.shape
+    for name, n in (("post", post), ("pre", pre)):
+        if n is not None:
+            _gpu(name + " weight", n[0], F32)
+            _need(n[0].shape == (D,), lambda: f"rms_norm_step: {name} {tuple(n[0].shape)}")
+    slots = wts = None
+    parts, top, isb = 1, 0, 0
+    more = (None, None, None)
+    if isinstance(y, ExpertTerms):
+        slots, wts, top = y.plan.slot_of_pair, y.weights, y.plan.top
+        more, y = (y.also, y.also_gate, y.rows), y.y
+        _gpu("y", y, F32)
+        _gpu("weights", wts, F32)
+        _need(y.dim() == 2 and y.shape[1] == D and wts.shape == (T, top)
+              and slots.shape[0] == T * top, "rms_norm_step: experts of another step")
+    elif y is not None:
+        _gpu("y", y, (F32, BF16))
+        isb = _is_bf16(y.dtype)
+        if y.dim() == 3:
+            _need(not isb, "rms_norm_step: partial sums are float32")
+            parts = y.shape[0]
+        _need(tuple(y.shape[-2:]) == (T, D) and y.dim() in (2, 3),
+              lambda: f"rms_norm_step: y {tuple(y.shape)} into {tuple(resid.shape)}")
+    n = T
+    if rows is not None:
+        _gpu("rows", rows, I32)
+        n = rows.shape[0]
+    out = None
+    if pre is not None:
+        out = torch.empty((n, D), dtype=rows_dtype, device=resid.device)
+    check(library("elementwise").kappai_rms_norm_step(
+        _ptr(resid), _ptr(y), _c_int(isb), _c_int(parts), _ptr(slots), _ptr(wts), _c_int(top),
+        *_terms_args("rms_norm_step", T, D, *more), _ptr(post[0] if post else None),
+        _c_float(post[1] if post else 0.0), _ptr(pre[0] if pre else None),
+        _c_float(pre[1] if pre else 0.0), _ptr(rows), _c_int(n), _c_int(T), _c_int(D), _ptr(out),
+        _c_int(_is_bf16(rows_dtype) if pre else 0), _stream()), "rms_norm_step")
+    return out
 
 
 # ---------------------------------------------------------------------------------------
@@ -1877,6 +1993,8 @@ def tanh_norm_step(resid: torch.Tensor, y=None, post: Optional[TanhNormWeights] 
                   lambda: f"tanh_norm_step: {name} {tuple(n.weight.shape)}, {tuple(n.bias.shape)}")
     slots = wts = None
     parts, top, isb = 1, 0, 0
+    if isinstance(y, ExpertTerms) and (y.also is not None or y.rows is not None):
+        y = y.combined()
     if isinstance(y, ExpertTerms):
         slots, wts, top, y = y.plan.slot_of_pair, y.weights, y.plan.top, y.y
         _gpu("y", y, F32)
@@ -2085,18 +2203,19 @@ def head_norm_rotate_store(proj: torch.Tensor, n_heads: int, n_kv_heads: int, di
                            rot_dims: int, rot_mode: int, k_pool: torch.Tensor,
                            v_pool: torch.Tensor, row_pos: torch.Tensor, row_seg: torch.Tensor,
                            block_tables: torch.Tensor, page_size: int,
-                           values_are_keys: bool = False) -> torch.Tensor:
+                           values_are_keys: bool = False, store_kv: bool = True) -> torch.Tensor:
     """From ``proj`` [T, H dim + G dim + G vdim (+ more)]: every q and k head divided by the root
     mean square of its own ``dim`` places and multiplied by a weight [dim] that the heads share
     (None: no norm), then the first ``rot_dims`` places turned by the row's position (tables and
     ``rot_mode`` as ``rotate_widen_store``).  Returns queries [T, H head_size] (zeros behind
     ``dim``); keys and values go to pools made for G kv heads of ``head_size``.
     ``values_are_keys``: there are no value columns; a kv head's value is its key as projected,
-    before norm and rotation."""
+    before norm and rotation.  ``store_kv`` False: ``proj`` holds queries only, and the pools are
+    left as they are (another layer's)."""
     H, G, d, dv, D = n_heads, n_kv_heads, dim, vdim, head_size
     _gpu("proj", proj, (F32, BF16), contiguous=False)
     T = proj.shape[0]
-    need = H * d + G * d + (0 if values_are_keys else G * dv)
+    need = H * d + (0 if not store_kv else G * d + (0 if values_are_keys else G * dv))
     _need(proj.dim() == 2 and proj.shape[1] >= need and proj.stride(1) == 1,
           lambda: f"head_norm_rotate_store: proj {tuple(proj.shape)} holds fewer than {need} "
                   "columns")
@@ -2125,7 +2244,8 @@ def head_norm_rotate_store(proj: torch.Tensor, n_heads: int, n_kv_heads: int, di
     q = torch.empty((T, H * D), dtype=proj.dtype, device=proj.device)
     check(library("attn_prep").kappai_head_norm_rotate_store(
         _ptr(proj), _c_int(proj.stride(0)), _ptr(q_norm_w), _ptr(k_norm_w), _c_float(eps),
-        _ptr(cos), _ptr(sin), _c_int(rot_dims), _c_int(rot_mode), _ptr(k_pool), _ptr(v_pool),
+        _ptr(cos), _ptr(sin), _c_int(rot_dims), _c_int(rot_mode), _ptr(k_pool if store_kv else None),
+        _ptr(v_pool if store_kv else None),
         _ptr(row_pos), _ptr(row_seg), _ptr(block_tables), _c_int(block_tables.shape[1]),
         _c_int(T), _c_int(H), _c_int(G), _c_int(d), _c_int(dv), _c_int(D), _c_int(page_size),
         _c_int(1 if values_are_keys else 0), _ptr(q), _c_int(_is_bf16(proj.dtype)), _stream()),
@@ -2415,14 +2535,83 @@ def matrix_state_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
     return out
 
 
+STATE_SPACE_CHUNK_ROWS = 128      # the most rows of a chunk the chunked form takes
+STATE_SPACE_MAX_STATE = 1024
+
+
+def state_space(xbc: torch.Tensor, z: torch.Tensor, n_heads: int, n_groups: int, dim: int,
+                vdim: int, z_bias: torch.Tensor, rate: torch.Tensor, skip: torch.Tensor,
+                state: torch.Tensor, seg_start: torch.Tensor, seg_pos0: torch.Tensor,
+                seg_slot: torch.Tensor, chunks: Optional[torch.Tensor] = None,
+                seg_chunk0: Optional[torch.Tensor] = None, chunk_rows: int = 0) -> torch.Tensor:
+    """A state ``S`` [vdim, dim] per head, float32, in ``state`` [slots, H, vdim, dim] (a segment that
+    starts at position 0 starts from zero), with one decay a head and token:
+    ``dt = softplus(z + z_bias[h])``, ``S <- exp(-rate[h] dt) S + x (dt B)^T``, ``y = S C + skip[h]
+    x``.  ``xbc`` [T, H vdim + 2 G dim]: x head by head, then B and C group by group (head h reads
+    group ``h // (H / G)``); ``z`` [T, >= H] in the same dtype (a view with a row stride);
+    ``z_bias``, ``rate``, ``skip`` [H] float32.  Returns y [T, H vdim] float32.
+
+    ``chunks`` [n, 3] = (segment, first row, rows <= ``chunk_rows``) with ``seg_chunk0`` [S + 1]: in
+    bfloat16, with sizes in multiples of eight, the rows are worked chunk by chunk in three passes
+    on the matrix cores (no chain along the tokens of a chunk; float32 operands go in as sums of
+    three bfloat16 values); else token by token."""
+    H, G, N, dv = n_heads, n_groups, dim, vdim
+    _gpu("xbc", xbc, (F32, BF16), contiguous=False)
+    _gpu("z", z, xbc.dtype, contiguous=False)
+    T = xbc.shape[0]
+    _need(H >= 1 and G >= 1 and H % G == 0 and 1 <= N <= STATE_SPACE_MAX_STATE,
+          lambda: f"state_space: {H} heads in {G} groups, a state of {N}")
+    _need(xbc.dim() == 2 and xbc.shape[1] >= H * dv + 2 * G * N and xbc.stride(1) == 1,
+          lambda: f"state_space: xbc {tuple(xbc.shape)} holds fewer than {H * dv + 2 * G * N} columns")
+    _need(z.dim() == 2 and z.shape[0] == T and z.shape[1] >= H and (z.stride(1) == 1 or H == 1),
+          lambda: f"state_space: z {tuple(z.shape)}")
+    for name, t in (("z_bias", z_bias), ("rate", rate), ("skip", skip)):
+        _gpu(name, t, F32)
+        _need(t.shape == (H,), lambda: f"state_space: {name} {tuple(t.shape)} for {H} heads")
+    _gpu("state", state, F32)
+    _need(tuple(state.shape[1:]) == (H, dv, N),
+          lambda: f"state_space: state {tuple(state.shape)} for {H} x {dv} x {N}")
+    for name, t in (("seg_start", seg_start), ("seg_pos0", seg_pos0), ("seg_slot", seg_slot)):
+        _gpu(name, t, I32)
+    S, dev = seg_slot.shape[0], xbc.device
+    b_at, c_at = H * dv, H * dv + G * N
+    out = torch.empty((T, H * dv), dtype=F32, device=dev)
+    lib = library("state_space")
+    at = (_c_int(xbc.stride(0)), _c_int(0), _c_int(b_at), _c_int(c_at))
+    consts = (_ptr(z), _c_int(z.stride(0)), _ptr(z_bias), _ptr(rate), _ptr(skip), _ptr(state))
+    if (chunks is not None and xbc.dtype == BF16
+            and lib.kappai_state_space_chunks_fit(_ptr(xbc), *at, _c_int(N), _c_int(dv))):
+        _gpu("chunks", chunks, I32)
+        _gpu("seg_chunk0", seg_chunk0, I32)
+        _need(chunks.dim() == 2 and chunks.shape[1] == 3 and seg_chunk0.shape[0] == S + 1
+              and 1 <= chunk_rows <= STATE_SPACE_CHUNK_ROWS,
+              lambda: f"state_space: chunk tables {tuple(chunks.shape)} of {chunk_rows} rows do not fit")
+        n_chunks = chunks.shape[0]
+        carry = torch.empty((n_chunks, H, dv, N), dtype=F32, device=dev)
+        total = torch.empty((n_chunks, H), dtype=F32, device=dev)
+        check(lib.kappai_state_space_chunks(
+            _ptr(xbc), *at, *consts, _ptr(seg_pos0), _ptr(seg_slot), _ptr(chunks),
+            _ptr(seg_chunk0), _c_int(n_chunks), _c_int(chunk_rows), _c_int(T), _c_int(S),
+            _c_int(H), _c_int(G), _c_int(N), _c_int(dv), _ptr(carry), _ptr(total), _ptr(out),
+            _stream()), "state_space_chunks")
+        return out
+    check(lib.kappai_state_space_walk(
+        _ptr(xbc), *at, *consts, _ptr(seg_start), _ptr(seg_pos0), _ptr(seg_slot), _c_int(T),
+        _c_int(S), _c_int(H), _c_int(G), _c_int(N), _c_int(dv), _ptr(out),
+        _c_int(_is_bf16(xbc.dtype)), _stream()), "state_space_walk")
+    return out
+
+
 GATE_SILU, GATE_SIGMOID = 0, 1
 
 
 def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor,
-                   gate_kind: int, n_heads: int, vdim: int, out_dtype) -> torch.Tensor:
+                   gate_kind: int, n_heads: int, vdim: int, out_dtype,
+                   gate_first: bool = False) -> torch.Tensor:
     """Per head ``o / sqrt(mean(o^2) + eps) * weight`` (``weight`` [vdim], shared by the heads, or
     [H, vdim], one a head) times ``silu(gate)`` or ``sigmoid(gate)``: ``o`` [T, H vdim] float32, ``gate`` [T, >= H vdim]
-    in ``out_dtype`` (a view with a row stride).  Returns [T, H vdim] in ``out_dtype``."""
+    in ``out_dtype`` (a view with a row stride).  ``gate_first``: the gate is applied before the
+    norm, whose mean it then enters.  Returns [T, H vdim] in ``out_dtype``."""
     H, dv = n_heads, vdim
     _gpu("o", o, F32)
     _gpu("weight", weight, F32)
@@ -2435,7 +2624,7 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, eps: float, gate: torc
     out = torch.empty((T, H * dv), dtype=out_dtype, device=o.device)
     check(library("linear_attention").kappai_head_norm_gate(
         _ptr(o), _ptr(weight), _c_float(eps), _ptr(gate), _c_int(gate.stride(0)),
-        _c_int(gate_kind), _c_int(T), _c_int(H), _c_int(dv),
+        _c_int(gate_kind), _c_int(1 if gate_first else 0), _c_int(T), _c_int(H), _c_int(dv),
         _c_int(dv if weight.dim() == 2 else 0), _ptr(out),
         _c_int(_is_bf16(out_dtype)), _stream()), "head_norm_gate")
     return out

@@ -70,3 +70,7 @@ LONE_ROWS_FROM = 4096
 # (chunk sums, carry over the chunks, outputs).
 SCAN_CHUNK_ROWS = 32
 SCAN_CHUNKS_FROM_ROWS = 64
+
+# The state-space recurrence: segments of up to this many rows are walked token by token, longer
+# ones (in bfloat16) worked in chunks on the matrix cores.
+STATE_SPACE_CHUNKS_FROM_ROWS = 16

@@ -12,6 +12,7 @@ from . import dukolorn  # noqa: F401  (registers Dukolorn)
 from . import lfm2  # noqa: F401  (registers Lfm2ForCausalLM)
 from . import nuzivik  # noqa: F401  (registers Nuzivik)
 from . import sibodra  # noqa: F401  (registers Sibodra)
+from . import zozezen  # noqa: F401  (registers Zozezen)
 from . import zumuzen  # noqa: F401  (registers Zumuzen)
 from .base import LayerCall, Model
 

@@ -22,6 +22,7 @@ from .positions import LearnedPositions
 from .rotary import RotaryEncoding, Rotation
 from .scored_attention import ScoredAttention
 from .shortconv import GatedShortConv
+from .state_space import StateSpaceDual
 
 __all__ = ["GroupedQueryAttention", "BLOCKS", "FEED_FORWARDS", "MIXERS", "NORMS",
            "POSITION_ENCODINGS", "Block", "FeedForward", "Hidden", "Mixer", "Norm", "Part",
@@ -31,4 +32,5 @@ __all__ = ["GroupedQueryAttention", "BLOCKS", "FEED_FORWARDS", "MIXERS", "NORMS"
            "ShortInputConv", "MinGRU", "MixtureOfExperts", "LearnedPositions", "OutputNormBlock",
            "LatentAttention", "GatedDeltaRule", "GatedLinearAttention", "ParallelMixer",
            "ScoredAttention", "RealGatedUnit", "BonusTimeMixing", "FixedDecayAttention",
-           "PassEntry", "HyperConnectionBlock", "LayerNorm", "SandwichNormBlock", "TanhNorm"]
+           "PassEntry", "HyperConnectionBlock", "LayerNorm", "SandwichNormBlock", "TanhNorm",
+           "StateSpaceDual"]

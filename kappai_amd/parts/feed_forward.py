@@ -27,22 +27,26 @@ class SwiGLU(FeedForward):
     takes_deferred_rows = True     # its first product takes what ops.linear takes
     adds_residual = True           # its last product can add into the residual stream
 
-    ACTIVATIONS = {"silu": ops.GLU_SILU, "gelu_tanh": ops.GLU_GELU_TANH}
+    ACTIVATIONS = {"silu": ops.GLU_SILU, "gelu_tanh": ops.GLU_GELU_TANH,
+                   "clamped": ops.GLU_CLAMPED}
 
     def __init__(self, prefix: str, width: int, hidden: int, dtype: torch.dtype, names=None,
                  activation: str = "silu", weight_suffix: str = ".weight", bias: bool = False,
-                 bias_suffix: str = ".bias"):
+                 bias_suffix: str = ".bias", clamp=None):
         """``activation``: what the gate passes through, "silu" or "gelu_tanh" (the tanh form of
-        GELU): ``W_down (act(W_gate x + b_gate) * (W_up x + b_up)) + b_down``; ``bias``: whether the
-        three maps have biases (the gate then runs as a kernel of its own behind the first
-        product, which adds the biases)."""
+        GELU): ``W_down (act(W_gate x + b_gate) * (W_up x + b_up)) + b_down``; or "clamped", the
+        clamped gate with the constants ``clamp`` (``ops.ClampedGate``).  ``bias``: whether the three
+        maps have biases.  With biases or the clamped gate the gate runs as a kernel of its own
+        behind the first product."""
         n = {"gate": "w1", "up": "w3", "down": "w2"}
         n.update(names or {})
         if activation not in self.ACTIVATIONS:
             raise ValueError(f"unknown gate activation {activation!r}; known: "
                              f"{', '.join(self.ACTIVATIONS)}")
+        if (activation == "clamped") != (clamp is not None):
+            raise ValueError(f"{prefix}: the clamped gate comes with its constants")
         self.width, self.hidden, self.dtype = width, hidden, dtype
-        self.activation = activation
+        self.activation, self.clamp = activation, clamp
         self.fused = False
         self.has_bias = bool(bias)
         self.gate_up = Linear([prefix + n["gate"], prefix + n["up"]], width, [hidden, hidden],
@@ -58,7 +62,7 @@ class SwiGLU(FeedForward):
         def interleaved(w):
             # the fused product wants gate and up rows in turns of 16
             self.fused = (w.dtype == torch.bfloat16 and self.hidden % ops.SWIGLU_GROUP == 0
-                          and self.width % 8 == 0 and not self.has_bias)
+                          and self.width % 8 == 0 and not self.has_bias and self.clamp is None)
             return ops.interleave_gate_up(w[:self.hidden], w[self.hidden:]) if self.fused else None
 
         self.gate_up.bind(tensors, arrange=interleaved)
@@ -73,7 +77,7 @@ class SwiGLU(FeedForward):
         gate_up = self.gate_up.forward(x)
         with profile.scope("ffn_act"):
             act = (ops.swiglu(gate_up) if self.activation == "silu"
-                   else ops.glu(gate_up, self.ACTIVATIONS[self.activation]))
+                   else ops.glu(gate_up, self.ACTIVATIONS[self.activation], self.clamp))
         return self.down.forward(act, partial_sums=not self.has_bias, add_into=into)
 
     def c_part(self, plan, view=None, shared_cache: bool = False):

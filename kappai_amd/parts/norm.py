@@ -15,6 +15,8 @@ from .cdesc import FoldDesc
 
 class RMSNorm(Norm):
     takes_partial_sums = True      # the kernel adds [S, T, width] partial sums itself, in order
+    takes_normed_update = True     # and RMS-norms a pending update on the way into the stream
+    takes_expert_terms = True      # and sums what a mixture's chosen experts left
     can_defer = True      # add_norm(..., defer=True) may hand out ops.ScaledRows or
                           # ops.FragmentRows in place of a tensor
 
@@ -47,6 +49,8 @@ class RMSNorm(Norm):
         a, sa, b, sb = y, 1.0, None, 1.0
         if isinstance(y, WeightedTerms):
             a, sa, b, sb = y.a, y.scale_a, y.b, y.scale_b
+        elif isinstance(y, ops.ExpertTerms):
+            a = y.combined()
         with profile.scope("rmsnorm"):
             return ops.output_norm_add(resid, a, self.weight, self.eps, rows_dtype=rows_dtype,
                                        scale_a=sa, b=b, scale_b=sb, add=add)
@@ -63,6 +67,13 @@ class RMSNorm(Norm):
         caller's next part takes what the product kernels take in place of the rows: such
         ``ops.ScaledRows`` as they are, or ``ops.FragmentRows`` (8 to 16 rows, made here in the
         order the product loads them)."""
+        if isinstance(delta, NormedUpdate):
+            if isinstance(delta.norm, RMSNorm) and self.width <= ops.RMS_STEP_MAX_WIDTH:
+                with profile.scope("rmsnorm" if rows is None else "logits_norm"):
+                    return ops.rms_norm_step(resid, delta.y, post=delta.norm.fold(),
+                                             pre=self.fold(), rows=rows, rows_dtype=self.dtype)
+            delta.norm.norm_output(resid, delta.y)
+            delta = None
         if isinstance(delta, ops.Added):
             if (defer and rows is None and isinstance(delta, ops.ScaledRows)
                     and delta.weight is self.weight and delta.eps == self.eps

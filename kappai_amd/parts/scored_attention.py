@@ -18,7 +18,10 @@ rotation; without ``head_norm_weight`` there is no such weight.  ``keep_first``:
 chunks) every position also sees the first ``keep_first`` positions of its sequence, at their true
 distance.  ``sink_value``: the sink is this constant score for every head (0: a one in the
 softmax's denominator) and no tensor.  ``head_gate``: a map ``W_g`` [heads, width] of the mixer's
-input gives one number a head, and the head's result is multiplied by its sigmoid before ``W_o``.
+input gives one number a head, and the head's result is multiplied by its sigmoid before ``W_o``.  ``own_keys`` False: the layer has no keys and values of
+its own (no ``W_k``, ``W_v``, key norm); it reads what another layer with the same heads, sizes and
+rotation keeps in the cache (a call of the schedule with ``reads_cache_of``), with its own queries,
+scale, gate and everything else.
 ``bucket``: a distance below half the
 table's rows has a row of its own; larger ones share rows on a logarithmic scale that reaches the
 last row at ``bias_max``.  Every piece is optional (``softcap`` 0, no table, no sink, no norm, no
@@ -76,7 +79,7 @@ class ScoredAttention(Mixer):
                  position=None, bias: bool = False, bias_suffix: str = ".bias",
                  values_from_keys: bool = False, head_qk_norm: bool = False,
                  sink_value: Optional[float] = None, head_gate: bool = False,
-                 head_norm_weight: bool = True, keep_first: int = 0):
+                 head_norm_weight: bool = True, keep_first: int = 0, own_keys: bool = True):
         n = {"q": "q", "k": "k", "v": "v", "o": "o", "q_norm": "q.norm", "k_norm": "k.norm",
              "rel": "rel", "sink": "sink", "gate": "g"}
         n.update(names or {})
@@ -116,9 +119,15 @@ class ScoredAttention(Mixer):
         if self.values_from_keys and vdim != dim:
             raise ValueError(f"{prefix}: values that are the keys have the keys' size {dim}, "
                              f"not {vdim}")
-        stacked = ["q", "k"] + ([] if self.values_from_keys else ["v"])
-        sizes = [num_heads * dim, num_kv_heads * dim] + (
-            [] if self.values_from_keys else [num_kv_heads * vdim])
+        self.own_keys = bool(own_keys)
+        if not self.own_keys and not self.head_qk_norm:
+            raise ValueError(f"{prefix}: keys of another layer go with the norm of every head by "
+                             "itself")
+        stacked, sizes = ["q"], [num_heads * dim]
+        if self.own_keys:
+            stacked, sizes = stacked + ["k"], sizes + [num_kv_heads * dim]
+            if not self.values_from_keys:
+                stacked, sizes = stacked + ["v"], sizes + [num_kv_heads * vdim]
         self._gate_at = sum(sizes)          # where the gates' columns start in the projection
         if self.head_gate:
             stacked.append("gate")
@@ -151,7 +160,8 @@ class ScoredAttention(Mixer):
             specs.append(TensorSpec(self._names["k_norm"], (self.G * self.d,), VECTOR, INIT_ONES))
         if self.head_qk_norm and self.head_norm_weight:
             specs.append(TensorSpec(self._names["q_norm"], (self.d,), VECTOR, INIT_ONES))
-            specs.append(TensorSpec(self._names["k_norm"], (self.d,), VECTOR, INIT_ONES))
+            if self.own_keys:
+                specs.append(TensorSpec(self._names["k_norm"], (self.d,), VECTOR, INIT_ONES))
         if self.bias_buckets:
             specs.append(TensorSpec(self._names["rel"], (self.bias_buckets, self.H), VECTOR,
                                     INIT_SMALL))
@@ -175,7 +185,8 @@ class ScoredAttention(Mixer):
                 self.d, dtype=torch.float32, device=tensors[self._o_name].device)
         elif self.whole_qk_norm or self.head_qk_norm:
             self.q_norm_w = tensors[self._names["q_norm"]].to(torch.float32).contiguous()
-            self.k_norm_w = tensors[self._names["k_norm"]].to(torch.float32).contiguous()
+            if self.own_keys:
+                self.k_norm_w = tensors[self._names["k_norm"]].to(torch.float32).contiguous()
         bias = sink = None
         if self.bias_buckets:
             bias = distance_bias_columns(tensors[self._names["rel"]], self.bias_far)
@@ -187,8 +198,9 @@ class ScoredAttention(Mixer):
         self.mods = ops.ScoreMods(self.softcap, bias, sink, self.keep_first)
 
     def forward(self, x, batch, cache, shared_cache: bool = False):
-        if shared_cache:
-            raise ValueError("this attention does not read another layer's keys")
+        if shared_cache == self.own_keys:
+            raise ValueError("this attention makes its own keys" if self.own_keys else
+                             "this attention reads another layer's keys and makes none")
         H, G, D = self.H, self.G, self.head_size
         proj = self.qkv.forward(x)
         tables = batch.block_tables[cache.group]
@@ -202,7 +214,7 @@ class ScoredAttention(Mixer):
                     rot.cos if rot else None, rot.sin if rot else None,
                     rot.rot_dim if rot else 0, rot.mode if rot else ops.ROT_NONE, k_pool, v_pool,
                     batch.row_pos, batch.row_seg, tables, cache.page_size,
-                    values_are_keys=self.values_from_keys)
+                    values_are_keys=self.values_from_keys, store_kv=self.own_keys)
             elif self.position is not None or self.values_from_keys:
                 rot = (self.position.rotation(x.device, batch.max_position)
                        if self.position is not None else None)

@@ -320,17 +320,18 @@ def scale_add_positions(x, scale, table, row_pos):
     x.mul_(scale).add_(table[row_pos.long()].to(F32))
 
 
-def glu(gate_up, kind):
+def glu(gate_up, kind, clamp=None):
     F = gate_up.shape[1] // 2
     g, u = gate_up[:, :F].to(F32), gate_up[:, F:].to(F32)
+    if kind == 2:
+        return _clamped(g, u, clamp).to(gate_up.dtype)
     if kind == 1:
-        a = 0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g ** 3)))
+        a = 0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g * g * g)))
     else:
         a = g / (1.0 + torch.exp(-g))
     return (a * u).to(gate_up.dtype)
 
 
-# ---- minGRU ----------------------------------------------------------------------------------
 def mingru_scan(proj, state, seg_start, seg_pos0, seg_slot, out_dtype, chunks=None,
                 seg_chunk0=None):
     proj = proj.to(F32)
@@ -571,13 +572,35 @@ def matrix_state_recurrence(q, k, v, z, n_heads, n_qk_heads, dim, vdim, rate, z_
     return out.reshape(T, H * dv)
 
 
-def head_norm_gate(o, weight, eps, gate, gate_kind, n_heads, vdim, out_dtype):
+def state_space(xbc, z, n_heads, n_groups, dim, vdim, z_bias, rate, skip, state, seg_start,
+                seg_pos0, seg_slot, chunks=None, seg_chunk0=None, chunk_rows=0):
+    H, G, N, dv = n_heads, n_groups, dim, vdim
+    T = xbc.shape[0]
+    x, B, C = xbc.to(F32).split([H * dv, G * N, G * N], dim=1)
+    x = x.reshape(T, H, dv)
+    B, C = (m.reshape(T, G, N).repeat_interleave(H // G, dim=1) for m in (B, C))
+    dt = torch.nn.functional.softplus(z[:, :H].to(F32) + z_bias)
+    out = torch.empty((T, H, dv), dtype=F32)
+    for s in range(seg_slot.shape[0]):
+        t0, t1, slot = int(seg_start[s]), int(seg_start[s + 1]), int(seg_slot[s])
+        S = torch.zeros((H, dv, N)) if int(seg_pos0[s]) == 0 else state[slot].clone()
+        for t in range(t0, t1):
+            S = (torch.exp(-rate * dt[t])[:, None, None] * S
+                 + (dt[t][:, None] * x[t])[:, :, None] * B[t][:, None, :])
+            out[t] = torch.einsum("hvn,hn->hv", S, C[t]) + skip[:, None] * x[t]
+        state[slot] = S
+    return out.reshape(T, H * dv)
+
+
+def head_norm_gate(o, weight, eps, gate, gate_kind, n_heads, vdim, out_dtype, gate_first=False):
     H, dv = n_heads, vdim
     T = o.shape[0]
     x = o.reshape(T, H, dv)
-    x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight        # [dv] or [H, dv]
     g = gate[:, :H * dv].to(F32).reshape(T, H, dv)
     g = g * torch.sigmoid(g) if gate_kind == GATE_SILU else torch.sigmoid(g)
+    if gate_first:
+        x, g = x * g, 1.0
+    x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight        # [dv] or [H, dv]
     return (x * g).reshape(T, H * dv).to(out_dtype)
 
 
@@ -690,22 +713,25 @@ def moe_route(x, router, top, bias=None):
     return chosen.to(torch.int32), torch.softmax(best, dim=-1)
 
 
-def moe_route_squashed(x, router, top, scale=1.0, correction=None, groups=1, keep_groups=1,
-                       bias=None):
+def moe_route_scored(x, router, top, scale=1.0, correction=None, groups=1, keep_groups=1,
+                     bias=None, score="sigmoid", group_best=2, gate=False):
     z = x.to(F32) @ router.T
+    if gate:
+        z, gates = z[:, :-1], torch.sigmoid(z[:, -1])
     if bias is not None:
         z = z + bias
-    s = torch.sigmoid(z)
+    s = torch.sigmoid(z) if score == "sigmoid" else torch.softmax(z, dim=-1)
     c = s if correction is None else s + correction
     T, E = s.shape
     if keep_groups < groups:
         by_group = c.reshape(T, groups, E // groups)
-        worth = by_group.topk(min(2, E // groups), dim=-1).values.sum(-1)
+        worth = by_group.topk(min(group_best, E // groups), dim=-1).values.sum(-1)
         kept = torch.zeros((T, groups), dtype=torch.bool)
         kept.scatter_(1, worth.topk(keep_groups, dim=-1).indices, True)
         c = by_group.masked_fill(~kept[:, :, None], -float("inf")).reshape(T, E)
     chosen = c.topk(top, dim=-1).indices
-    return chosen.to(torch.int32), s.gather(1, chosen) * scale
+    out = chosen.to(torch.int32), s.gather(1, chosen) * scale
+    return (*out, gates) if gate else out
 
 
 def tanh_norm_step(resid, y=None, post=None, pre=None, rows=None, rows_dtype=None):
@@ -732,24 +758,32 @@ def moe_plan(experts, n_experts):
     return _Plan(experts)
 
 
-def moe_experts_gated(x, w_gate, w_up, plan):
+def _clamped(g, u, c):
+    g = g.clamp(max=c.limit)
+    return g * torch.sigmoid(c.slope * g) * (u.clamp(-c.limit, c.limit) + c.shift)
+
+
+# (what belongs to experts without matrices stays NaN: nothing may read it)
+def moe_experts_gated(x, w_gate, w_up, plan, clamp=None):
     T, top = plan.experts.shape
-    out = torch.empty((T, top, w_gate.shape[1]), dtype=x.dtype)
-    for t in range(T):
-        for k in range(top):
-            e = int(plan.experts[t, k])
-            g = w_gate[e].to(F32) @ x[t].to(F32)
-            u = w_up[e].to(F32) @ x[t].to(F32)
-            out[t, k] = (g / (1.0 + torch.exp(-g)) * u).to(x.dtype)
+    out = torch.full((T, top, w_gate.shape[1]), float("nan"), dtype=x.dtype)
+    for e in range(w_gate.shape[0]):
+        t, k = (plan.experts == e).nonzero(as_tuple=True)
+        if not len(t):
+            continue
+        g = x[t].to(F32) @ w_gate[e].to(F32).T
+        u = x[t].to(F32) @ w_up[e].to(F32).T
+        out[t, k] = (_clamped(g, u, clamp) if clamp else g / (1.0 + torch.exp(-g)) * u).to(x.dtype)
     return out
 
 
 def moe_experts_down(act, w_down, plan):
     T, top = plan.experts.shape
-    out = torch.empty((T, top, w_down.shape[1]), dtype=F32)
-    for t in range(T):
-        for k in range(top):
-            out[t, k] = w_down[int(plan.experts[t, k])].to(F32) @ act[t, k].to(F32)
+    out = torch.full((T, top, w_down.shape[1]), float("nan"), dtype=F32)
+    for e in range(w_down.shape[0]):
+        t, k = (plan.experts == e).nonzero(as_tuple=True)
+        if len(t):
+            out[t, k] = act[t, k].to(F32) @ w_down[e].to(F32).T
     return out
 
 
@@ -763,22 +797,55 @@ def moe_experts_activated(x, w_up, plan):
     return out
 
 
-def moe_combine(y, weights, plan, also=None):
+def moe_combine(y, weights, plan, also=None, also_gate=None, rows=None):
+    if rows is not None:
+        handed_on = y.isnan().any(dim=-1, keepdim=True)
+        y = torch.where(handed_on, rows.to(F32)[:, None, :], y)
     out = (y * weights[:, :, None]).sum(dim=1)
     if also is not None:
+        more = torch.zeros_like(out)
         for p in (also if also.dim() == 3 else also[None]):
-            out = out + p.to(F32)
+            more = more + p.to(F32)
+        out = out + (more if also_gate is None else more * also_gate[:, None])
     return out
+
+
+RMS_STEP_MAX_WIDTH = 8192
+
+
+def rms_norm_step(resid, y=None, post=None, pre=None, rows=None, rows_dtype=None):
+    def n_of(x, n):
+        return x / torch.sqrt((x * x).mean(-1, keepdim=True) + n[1]) * n[0]
+
+    x = resid
+    if y is not None:
+        if hasattr(y, "combined"):
+            y = y.combined()
+        u = torch.zeros_like(resid)
+        for p in (y if y.dim() == 3 else y[None]):
+            u = u + p.to(F32)
+        x = resid + (n_of(u, post) if post is not None else u)
+        if rows is None:
+            resid.copy_(x)
+    if pre is None:
+        return None
+    return n_of(x if rows is None else x[rows.long()], pre).to(rows_dtype)
 
 
 def head_norm_rotate_store(proj, n_heads, n_kv_heads, dim, vdim, head_size, q_norm_w, k_norm_w,
                            eps, cos, sin, rot_dims, rot_mode, k_pool, v_pool, row_pos, row_seg,
-                           block_tables, page_size, values_are_keys=False):
+                           block_tables, page_size, values_are_keys=False, store_kv=True):
     H, G, d, dv, D = n_heads, n_kv_heads, dim, vdim, head_size
     T = proj.shape[0]
     p = proj.to(F32)
     pos = row_pos.long()
     q = p[:, :H * d].reshape(T, H, d)
+    if not store_kv:
+        if q_norm_w is not None:
+            q = q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * q_norm_w
+        qo = torch.zeros((T, H, D), dtype=F32)
+        qo[:, :, :d] = _rotate(q, pos, cos, sin, rot_dims, rot_mode)
+        return qo.reshape(T, H * D).to(proj.dtype)
     k = p[:, H * d:(H + G) * d].reshape(T, G, d)
     v = k if values_are_keys else p[:, (H + G) * d:(H + G) * d + G * dv].reshape(T, G, dv)
     if q_norm_w is not None:
@@ -840,7 +907,7 @@ def activate(x, kind=0):
     return (r * r).to(x.dtype)
 
 
-ALL = ["moe_route_squashed", "tanh_norm_step", "moe_experts_activated", "head_norm_rotate_store", "hyper_step", "rows_rmsnorm", "sigmoid_gate",
+ALL = ["moe_route_scored", "rms_norm_step", "state_space", "tanh_norm_step", "moe_experts_activated", "head_norm_rotate_store", "hyper_step", "rows_rmsnorm", "sigmoid_gate",
        "softcap_rows", "activate", "add_group_rmsnorm", "add_group_rmsnorm_canon_step", "canon_conv", "scale_add_positions", "glu", "mingru_scan", "diff_store",
        "diff_combine", "moe_route", "moe_plan", "moe_experts_gated", "moe_experts_down", "moe_combine",
        "output_norm_add", "projection_norm_store", "latent_store", "headwise_linear", "conv_silu",

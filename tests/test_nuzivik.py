@@ -225,7 +225,7 @@ def test_plain_choice_by_groups_with_negative_scores():
     router = {"experts": 4, "top": 2, "groups": {"count": 2, "keep": 1}}
     order, gap = P.choose(s, corr, router)
     assert order == [2, 3] and gap == pytest.approx(min(-1.0 - (-2.0), math.inf))
-    chosen, wts = emulated_ops.moe_route_squashed(
+    chosen, wts = emulated_ops.moe_route_scored(
         torch.log(s / (1 - s)).float()[None], torch.eye(4), 2, 1.5, correction=corr.float(),
         groups=2, keep_groups=1)
     assert sorted(chosen[0].tolist()) == [2, 3] and torch.allclose(wts, torch.tensor([[0.75, 0.75]]))

@@ -220,7 +220,7 @@ def test_squashed_router(dtype, W, E, top, groups, keep, scale, T):
     cfg = {"experts": E, "top": top, "groups": {"count": groups, "keep": keep}}
     s = torch.sigmoid(x.double() @ router.double().T)
     for c in (corr, None):
-        chosen, wts = ops.moe_route_squashed(x.to(DEV), router.to(DEV), top, scale,
+        chosen, wts = ops.moe_route_scored(x.to(DEV), router.to(DEV), top, scale,
                                              correction=None if c is None else c.to(DEV),
                                              groups=groups, keep_groups=keep)
         chosen, wts = chosen.cpu(), wts.cpu().double()
@@ -235,11 +235,11 @@ def test_squashed_router(dtype, W, E, top, groups, keep, scale, T):
             assert all(abs(got[e] - float(s[i, e]) * scale) < 1e-5 * scale for e in order)
         assert clear >= 0.9 * T
     bias = torch.randn(E, generator=g)
-    chosen, wts = ops.moe_route_squashed(x.to(DEV), router.to(DEV), top, bias=bias.to(DEV))
+    chosen, wts = ops.moe_route_scored(x.to(DEV), router.to(DEV), top, bias=bias.to(DEV))
     want = torch.sigmoid(x.double() @ router.double().T + bias.double())
     assert rel(wts, want.gather(1, chosen.cpu().long())) < 1e-5
     with pytest.raises(ValueError, match="groups"):
-        ops.moe_route_squashed(x.to(DEV), router.to(DEV), top, groups=E + 1)
+        ops.moe_route_scored(x.to(DEV), router.to(DEV), top, groups=E + 1)
 
 
 def dense_attention(q, k, v, pos, window, chunk, keep, scale, table, sink, cap=0.0):
