@@ -121,7 +121,12 @@ COMPARISONS = {"w1024": ("dapipel-w1024", "lfm2-like-w1024"),
                # the Nuzivik decoder beside the Sibodra decoder of equal size (its closest
                # relative: the same scored attention, a mixture of experts) and the LFM2 shapes
                "nuzivik-w1024": ("nuzivik-w1024", "sibodra-w1024", "lfm2-like-w1024"),
-               "nuzivik-w2048": ("nuzivik-w2048", "sibodra-w2048", "lfm2-like-w2048")}
+               "nuzivik-w2048": ("nuzivik-w2048", "sibodra-w2048", "lfm2-like-w2048"),
+               # the Zozezen decoder beside the Nuzivik decoder of equal size (its closest
+               # relative: norms on both sides of a sublayer, scored attention, a mixture of
+               # experts in groups) and the Zumuzen decoder (a state per head worked in chunks)
+               "zozezen-w1024": ("zozezen-w1024", "nuzivik-w1024", "zumuzen-w1024"),
+               "zozezen-w2048": ("zozezen-w2048", "nuzivik-w2048", "zumuzen-w2048")}
 
 
 def stage_table(runner, entries_of, reps):
@@ -580,13 +585,13 @@ def main() -> int:
                          "the greedy choice (1: none)")
     ap.add_argument("--compare", default="", metavar="SIZES",
                     help="instead of the headline run: prompt and decode steps of the Dapipel, "
-                         "Dukolorn, Zumuzen, Sibodra or Nuzivik decoder beside the LFM2 shape of "
+                         "Dukolorn, Zumuzen, Sibodra, Nuzivik or Zozezen decoder beside models of "
                          "equal size, at these sizes (comma separated: " + ", ".join(sorted(COMPARISONS)) + "; 'all')")
     args = ap.parse_args()
     if args.compare:
         keys = (sorted(k for k in COMPARISONS if k.startswith("w")) if args.compare == "all"
                 else sorted(k for k in COMPARISONS if k.startswith(args.compare + "-"))
-                if args.compare in ("dukolorn", "zumuzen", "sibodra", "nuzivik")
+                if args.compare in ("dukolorn", "zumuzen", "sibodra", "nuzivik", "zozezen")
                 else args.compare.split(","))
         for k in keys:
             if k not in COMPARISONS:

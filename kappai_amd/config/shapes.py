@@ -271,6 +271,53 @@ SHAPES.update({
 })
 
 
+def _zozezen(width, mixers, heads, kv_heads, dim, vdim, m_heads, m_vdim, state, m_groups,
+             norm_groups, ff, experts, identity, top, groups, keep_groups, limit=7.0,
+             vocab=65536) -> dict:
+    """Layers by letter: "m" a state-space mixer, "a" an attention with keys of its own, "s" one
+    that reads the last "a" layer's; a mixture of ``experts`` experts of ``ff // top`` and ``identity``
+    that hand their input on, in groups, with a shared expert of the same size, everywhere."""
+    mlp = {"kind": "moe", "expert": {"ff": ff // top, "limit": limit},
+           "shared": {"ff": ff // top, "limit": limit},
+           "router": {"experts": experts, "identity": identity, "top": top,
+                      "groups": {"count": groups, "keep": keep_groups}}}
+    layers, source = [], None
+    for i, kind in enumerate(mixers):
+        if kind == "m":
+            layers.append({"type": "mamba2",
+                           "mixer": {"heads": m_heads, "vdim": m_vdim, "state": state,
+                                     "groups": m_groups, "conv": 4, "norm_groups": norm_groups}})
+        else:
+            mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+                     "scale": dim ** -0.5, "rot": {"base": 1000000.0, "dims": dim}}
+            if kind == "s":
+                mixer["kv_from"] = source
+            else:
+                source = i
+            layers.append({"type": "attention", "mixer": mixer})
+        layers[-1]["mlp"] = copy.deepcopy(mlp)
+    return {"architecture": "Zozezen", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+            "layers": layers}
+
+
+SHAPES.update({
+    # eight layers at a width of 1024, state-space mixers and attention in turns, every second
+    # attention on the keys of the one before: 32 state-space heads of 64 with a state of 128 in 4
+    # groups, 16 attention heads of 64 on 4 kv heads; 16 experts of 1152 and 4 that hand their
+    # input on, in 4 groups of which 2 can be chosen from, 4 a token (4608 active at most), beside
+    # a shared one
+    "zozezen-w1024": _zozezen(1024, "mamsmams", 16, 4, 64, 64, 32, 64, 128, 4, 4, 4608, 16, 4, 4,
+                              4, 2),
+    # the same at a width of 2048: 64 state-space heads in 8 groups, 32 attention heads on 8 kv
+    # heads, experts of 2048 (8192 active at most)
+    "zozezen-w2048": _zozezen(2048, "mamsmams", 32, 8, 64, 64, 64, 64, 128, 8, 8, 8192, 16, 4, 4,
+                              4, 2),
+    # a tiny one for smoke runs
+    "zozezen-tiny": _zozezen(64, "mas", 4, 2, 16, 8, 4, 8, 16, 2, 1, 96, 6, 2, 2, 2, 1, limit=2.0,
+                             vocab=256),
+})
+
+
 def named_shape(name: str) -> dict:
     """A copy of the configuration called ``name`` (any case), or a ``KeyError`` naming them all."""
     key = name.strip().lower()
