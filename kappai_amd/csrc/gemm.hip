@@ -127,7 +127,9 @@ __device__ __forceinline__ void store_out(bf16_t* p, float v) { *p = f32_to_bf16
 // g < -88: the reciprocal is then 0 and the result -0, as it should be.
 // GATE_ACT (a constant of the build) chooses what the gated epilogues pass the gate through:
 // 0 silu; 1 the tanh form of gelu, 0.5 g (1 + tanh(a)) with a = sqrt(2/pi) (g + 0.044715 g^3),
-// which is g * sigmoid(2 a) and so the same two instructions.
+// which is g * sigmoid(2 a) and so the same two instructions; 2 the clamped gate, g = min(g, limit),
+// u = clamp(u, -limit, limit), g sigmoid(slope g) (u + shift), whose three constants the gated
+// epilogues read where the others find a bias (a gated product has none).
 #ifndef GATE_ACT
 #define GATE_ACT 0
 #endif
@@ -137,6 +139,19 @@ __device__ __forceinline__ float silu_f(float g) {
   return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * a2));
 #else
   return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * g));
+#endif
+}
+
+// What a gated epilogue makes of the sums of a gate row and an up row.
+__device__ __forceinline__ float gated_f(float g, float u, const float* __restrict__ consts) {
+#if GATE_ACT == 2
+  const float limit = consts[0], slope = consts[1], shift = consts[2];
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * slope * g)) *
+         (u + shift);
+#else
+  return silu_f(g) * u;
 #endif
 }
 
@@ -305,7 +320,7 @@ __global__ __launch_bounds__(WAVES_M * WAVES_N * WAVE)
           const float other = __shfl_xor(acc[i][j][v], 16, WAVE);
           const int gm = m0 + (wm * WM + i) * 32 + 8 * (v / 4) + 4 * (lane / 32) + v % 4;
           if (c < 16 && gm < M && gcol + c < N)
-            store_out(C + (size_t)gm * ldc + on, silu_f(acc[i][j][v]) * other);
+            store_out(C + (size_t)gm * ldc + on, gated_f(acc[i][j][v], other, bias));
         }
       }
     return;
@@ -650,7 +665,8 @@ void gemm_bf16_block256_kernel(const bf16_t* __restrict__ A, const bf16_t* __res
         if (EPI == 1) {
           c = j * 16 + 8 * g + 4 * hh;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v4[e] = silu_f(acc[i][j][4 * g + e]) * acc[i][j][4 * g + 8 + e];
+          for (int e = 0; e < 4; ++e)
+            v4[e] = gated_f(acc[i][j][4 * g + e], acc[i][j][4 * g + 8 + e], bias);
         } else {
           c = j * 32 + 8 * g + 4 * hh;
 #pragma unroll
@@ -1042,7 +1058,7 @@ __global__ __launch_bounds__((NW < 16 ? NW + 1 : NW) * WAVE) void gemm_bf16_skin
     }
   } else if (wave < MT && gn < N && (EPI != 3 || col < 8)) {
     const int t = wave;
-    const float bv = (bias && blockIdx.y == 0) ? bias[gn] : 0.f;
+    const float bv = (EPI != 1 && bias && blockIdx.y == 0) ? bias[gn] : 0.f;
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
       const int gm = t * 16 + 4 * (lane / 16) + v;
@@ -1056,7 +1072,7 @@ __global__ __launch_bounds__((NW < 16 ? NW + 1 : NW) * WAVE) void gemm_bf16_skin
           float up = red[0][MT + t][lane][v];
 #pragma unroll
           for (int w = 1; w < NW; ++w) up += red[w][MT + t][lane][v];
-          store_out(C + out_at(gm, gn), silu_f(sum) * (up * rs));
+          store_out(C + out_at(gm, gn), gated_f(sum, up * rs, bias));
         } else if (EPI == 2 || EPI == 3) {
           // where the other two gates of this channel lie: EPI 2 in row groups 1 and 2 of this
           // lane, EPI 3 the C gate 8 columns further in group 0 and the x gate in group 1
@@ -1464,7 +1480,7 @@ __global__ __launch_bounds__(NWN * NWK * WAVE) void gemm_bf16_shared_rows_kernel
       if (EPI == 1) {
         const int on = wrow0 / 2 + col;                 // 16 output columns a wave
         if (wrow0 + 16 + col < n_rows_w)
-          store_out(C + (size_t)gm * ldc + on, silu_f(sum[0][v]) * sum[1][v]);
+          store_out(C + (size_t)gm * ldc + on, gated_f(sum[0][v], sum[1][v], bias));
       } else {
 #pragma unroll
         for (int r = 0; r < 2; ++r) {
@@ -1686,10 +1702,10 @@ __global__ __launch_bounds__(R32_NWN * R32_NWK * WAVE) void gemm_bf16_rows32_ker
 #pragma unroll
         for (int g = 0; g < 2; ++g) {
           uint2 pk;
-          pk.x = pack_bf16x2(silu_f(sum[4 * g]) * sum[4 * g + 8],
-                             silu_f(sum[4 * g + 1]) * sum[4 * g + 9]);
-          pk.y = pack_bf16x2(silu_f(sum[4 * g + 2]) * sum[4 * g + 10],
-                             silu_f(sum[4 * g + 3]) * sum[4 * g + 11]);
+          pk.x = pack_bf16x2(gated_f(sum[4 * g], sum[4 * g + 8], bias),
+                             gated_f(sum[4 * g + 1], sum[4 * g + 9], bias));
+          pk.y = pack_bf16x2(gated_f(sum[4 * g + 2], sum[4 * g + 10], bias),
+                             gated_f(sum[4 * g + 3], sum[4 * g + 11], bias));
           if constexpr (sizeof(TO) == 2)
             *reinterpret_cast<uint2*>(C + (size_t)gm * ldc + wrow0 / 2 + 8 * g + 4 * hh) = pk;
         }
@@ -1892,20 +1908,30 @@ extern "C" int kappai_gemm_bf16(const void* A, const void* W, const void* W_frag
 }
 
 // C[M, F] = silu(A Wg^T) * (A Wu^T) with W = gate and up rows interleaved in groups of 16,
-// [2F, K]; F must be a multiple of 16.
-extern "C" int kappai_gemm_bf16_swiglu(const void* A, const void* W, const void* W_frag, void* C,
-                                       int M, int F, int K, int lda, int ldc, int force_kernel,
-                                       int a_frag, const float* scale_ss, int scale_parts,
-                                       float scale_eps, int c_frag, hipStream_t stream) {
+// [2F, K]; F must be a multiple of 16.  `consts`: the gate's constants, where GATE_ACT has any.
+extern "C" int kappai_gemm_bf16_gated(const void* A, const void* W, const void* W_frag, void* C,
+                                      int M, int F, int K, int lda, int ldc, int force_kernel,
+                                      int a_frag, const float* scale_ss, int scale_parts,
+                                      float scale_eps, int c_frag, const float* consts,
+                                      hipStream_t stream) {
   if (M <= 0 || F <= 0) return 0;
+  if ((consts != nullptr) != (GATE_ACT == 2)) return (int)hipErrorInvalidValue;
   if ((K % 8) || (lda % 8) || (F % 16)) return (int)hipErrorInvalidValue;
   if (force_kernel == 2 && M > 64) return (int)hipErrorInvalidValue;
   if (!frag_ok(W_frag, 2 * F, K) || (a_frag && (K % 32))) return (int)hipErrorInvalidValue;
   Fuse fuse{RowScale{scale_ss, scale_parts, scale_eps}, ResidOut{}, c_frag};
   if (!fuse_ok(fuse, M, F, K, 0, 1)) return (int)hipErrorInvalidValue;
-  return launch_bf16<bf16_t, 1>((const bf16_t*)A, (const bf16_t*)W, nullptr, (bf16_t*)C, M, F, K,
+  return launch_bf16<bf16_t, 1>((const bf16_t*)A, (const bf16_t*)W, consts, (bf16_t*)C, M, F, K,
                                 lda, ldc, force_kernel, 1, stream, ConvStep{},
                                 (const bf16_t*)W_frag, a_frag, fuse);
+}
+
+extern "C" int kappai_gemm_bf16_swiglu(const void* A, const void* W, const void* W_frag, void* C,
+                                       int M, int F, int K, int lda, int ldc, int force_kernel,
+                                       int a_frag, const float* scale_ss, int scale_parts,
+                                       float scale_eps, int c_frag, hipStream_t stream) {
+  return kappai_gemm_bf16_gated(A, W, W_frag, C, M, F, K, lda, ldc, force_kernel, a_frag, scale_ss,
+                                scale_parts, scale_eps, c_frag, nullptr, stream);
 }
 
 // Conv layer decode step in one kernel: C[M, D] = Cgate * conv(Bgate * x | state) from A [M, K]

@@ -21,7 +21,7 @@
 
 extern "C" int kappai_moe_tile_rows() { return MOE_TILE_M; }
 
-#define MOE_ROUTE_GROUP 16      // experts whose sums a thread carries side by side
+#define MOE_ROUTE_GROUP 8       // experts whose sums a thread carries side by side
 
 // How a router that scores every expert chooses: score s = sigmoid(z) of its own logit (over_all
 // 0) or softmax(z) over all experts (1), choice score s + correction[e] (null: s).  The experts form
@@ -82,64 +82,89 @@ __device__ __forceinline__ void moe_score(const moe_scored_choice& c, int E, flo
   meet();
 }
 
-// A block a row.  The threads stride over the row four columns at a time (one column at a time
-// when the width or an address does not allow 16-byte loads), each with the sums of a group of
-// experts, whose loads are all asked for before the first is used; the waves' sums meet in LDS
-// and are added in the order of the waves.  Then the first wave chooses.  `gates` (null: none): the
-// router holds one more row behind the E experts', and sigmoid of its logit is the row's gate.
-template <typename T, int VEC, bool SCORED>
-__global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
+// ROWS rows a block.  The waves form teams; a team strides over the columns four at a time (one at a
+// time when the width or an address does not allow 16-byte loads) with the sums of a group of
+// experts, whose loads are all asked for before the first is used; the teams take the groups in
+// turns.  A team's sums meet in LDS and are added in the order of its waves.  Then wave r chooses for
+// row r.  Few rows: one a block, wide blocks of several teams, so that all of the router is asked for
+// at once; many: several a block, which read the router together.  `gates` (null: none): the router
+// holds one more row behind the E experts', and sigmoid of its logit is the row's gate.
+template <typename T, int VEC, bool SCORED, int THREADS, int ROWS>
+__global__ __launch_bounds__(THREADS) void moe_route_kernel(
     const T* __restrict__ x, int ldx, const float* __restrict__ router,
-    const float* __restrict__ bias, int n_rows, int D, int E, int top, moe_scored_choice sq,
-    float* __restrict__ gates, int* __restrict__ idx, float* __restrict__ wts) {
+    const float* __restrict__ bias, int n_rows, int D, int E, int top, int teams,
+    moe_scored_choice sq, float* __restrict__ gates, int* __restrict__ idx,
+    float* __restrict__ wts) {
   extern __shared__ float route_lds[];
-  constexpr int NW = MOE_THREADS / WAVE;
+  constexpr int NW = THREADS / WAVE;
   const int n_logits = gates != nullptr ? E + 1 : E;
-  float* logits = route_lds;                       // [n_logits]
-  float* part = route_lds + n_logits;              // [MOE_ROUTE_GROUP][NW]
+  const int per_row = n_logits + (SCORED ? E + sq.groups : 0);
+  float* part = route_lds + ROWS * per_row;        // [ROWS][MOE_ROUTE_GROUP][NW]
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-  const int row = blockIdx.x;
-  const T* xr = x + (size_t)row * ldx;
-  for (int e0 = 0; e0 < n_logits; e0 += MOE_ROUTE_GROUP) {
-    float acc[MOE_ROUTE_GROUP];
+  const int row0 = blockIdx.x * ROWS;
+  const int team_threads = THREADS / teams, team_waves = NW / teams;
+  const int team = threadIdx.x / team_threads, tid = threadIdx.x % team_threads;
+  const T* xr[ROWS];
 #pragma unroll
-    for (int j = 0; j < MOE_ROUTE_GROUP; ++j) acc[j] = 0.f;
-    for (int c = threadIdx.x * VEC; c < D; c += MOE_THREADS * VEC) {
-      float xv[VEC], rv[MOE_ROUTE_GROUP][VEC];
+  for (int r = 0; r < ROWS; ++r) xr[r] = x + (size_t)min(row0 + r, n_rows - 1) * ldx;
+  for (int e00 = 0; e00 < n_logits; e00 += MOE_ROUTE_GROUP * teams) {
+    const int e0 = e00 + MOE_ROUTE_GROUP * team;
+    if (e0 < n_logits) {
+      float acc[ROWS][MOE_ROUTE_GROUP];
 #pragma unroll
-      for (int j = 0; j < MOE_ROUTE_GROUP; ++j) {
-        const float* r = router + (size_t)min(e0 + j, n_logits - 1) * D + c;
-        if (VEC == 4) {
-          const float4 v = *reinterpret_cast<const float4*>(r);
-          rv[j][0] = v.x; rv[j][VEC > 1 ? 1 : 0] = v.y; rv[j][VEC > 2 ? 2 : 0] = v.z;
-          rv[j][VEC > 3 ? 3 : 0] = v.w;
-        } else {
-          rv[j][0] = r[0];
+      for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+        for (int j = 0; j < MOE_ROUTE_GROUP; ++j) acc[r][j] = 0.f;
+      for (int c = tid * VEC; c < D; c += team_threads * VEC) {
+        float xv[ROWS][VEC], rv[MOE_ROUTE_GROUP][VEC];
+#pragma unroll
+        for (int j = 0; j < MOE_ROUTE_GROUP; ++j) {
+          const float* w = router + (size_t)min(e0 + j, n_logits - 1) * D + c;
+          if (VEC == 4) {
+            const float4 v = *reinterpret_cast<const float4*>(w);
+            rv[j][0] = v.x; rv[j][VEC > 1 ? 1 : 0] = v.y; rv[j][VEC > 2 ? 2 : 0] = v.z;
+            rv[j][VEC > 3 ? 3 : 0] = v.w;
+          } else {
+            rv[j][0] = w[0];
+          }
         }
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+          for (int i = 0; i < VEC; ++i) xv[r][i] = to_f32(xr[r][c + i]);
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+          for (int j = 0; j < MOE_ROUTE_GROUP; ++j)
+#pragma unroll
+            for (int i = 0; i < VEC; ++i) acc[r][j] = fmaf(xv[r][i], rv[j][i], acc[r][j]);
       }
 #pragma unroll
-      for (int i = 0; i < VEC; ++i) xv[i] = to_f32(xr[c + i]);
+      for (int r = 0; r < ROWS; ++r)
 #pragma unroll
-      for (int j = 0; j < MOE_ROUTE_GROUP; ++j)
-#pragma unroll
-        for (int i = 0; i < VEC; ++i) acc[j] = fmaf(xv[i], rv[j][i], acc[j]);
-    }
-#pragma unroll
-    for (int j = 0; j < MOE_ROUTE_GROUP; ++j) {
-      const float sum = wave_sum(acc[j]);
-      if (lane == 0) part[j * NW + wave] = sum;
+        for (int j = 0; j < MOE_ROUTE_GROUP; ++j) {
+          const float sum = wave_sum(acc[r][j]);
+          if (lane == 0) part[(r * MOE_ROUTE_GROUP + j) * NW + wave] = sum;
+        }
     }
     __syncthreads();
-    if (threadIdx.x < MOE_ROUTE_GROUP && e0 + threadIdx.x < n_logits) {
-      float sum = part[threadIdx.x * NW];
-      for (int w = 1; w < NW; ++w) sum += part[threadIdx.x * NW + w];
-      logits[e0 + threadIdx.x] = bias && e0 + threadIdx.x < E ? sum + bias[e0 + threadIdx.x] : sum;
+    for (int i = threadIdx.x; i < ROWS * MOE_ROUTE_GROUP * teams; i += THREADS) {
+      const int j = i % MOE_ROUTE_GROUP, tm = (i / MOE_ROUTE_GROUP) % teams;
+      const int r = i / (MOE_ROUTE_GROUP * teams), e = e00 + MOE_ROUTE_GROUP * tm + j;
+      if (e < n_logits) {
+        const float* p = part + (r * MOE_ROUTE_GROUP + j) * NW + tm * team_waves;
+        float sum = p[0];
+        for (int w = 1; w < team_waves; ++w) sum += p[w];
+        route_lds[r * per_row + e] = bias && e < E ? sum + bias[e] : sum;
+      }
     }
     __syncthreads();
   }
-  if (wave != 0) return;
+  const int row = row0 + wave;
+  if (wave >= ROWS || row >= n_rows) return;
+  float* logits = route_lds + wave * per_row;      // [n_logits]
+  float* score = logits + n_logits;                // [E], then [groups] (scored choice only)
   if (gates != nullptr && lane == 0) gates[row] = 1.0f / (1.0f + expf(-logits[E]));
-  float* score = part + MOE_ROUTE_GROUP * NW;      // [E], then [groups] (scored choice only)
   if (SCORED) moe_score(sq, E, logits, score, score + E);
   float cv[MOE_MAX_TOP];
   int ci[MOE_MAX_TOP];
@@ -186,6 +211,10 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_route_kernel(
   }
 }
 
+#define MOE_ROUTE_WIDE 1024         // threads of a block that takes one row
+#define MOE_ROUTE_SHARED_ROWS 4     // rows of a block of MOE_THREADS
+#define MOE_ROUTE_WIDE_ROWS 512     // up to this many rows of a step take a wide block each
+
 static int moe_route_launch(const void* x, int ldx, int x_is_bf16, const float* router,
                             const float* bias, int T, int D, int E, int top, bool scored,
                             moe_scored_choice sq, float* gates, int* idx, float* wts,
@@ -195,19 +224,33 @@ static int moe_route_launch(const void* x, int ldx, int x_is_bf16, const float* 
   if (scored && (sq.groups < 1 || sq.keep < 1 || sq.keep > sq.groups || E % sq.groups ||
                  top > E / sq.groups * sq.keep || sq.best < 1 || sq.best > 2))
     return (int)hipErrorInvalidValue;
-  const size_t lds = ((size_t)E + 1 + MOE_ROUTE_GROUP * (MOE_THREADS / WAVE) +
-                      (scored ? E + sq.groups : 0)) * sizeof(float);
+  const int n_logits = gates ? E + 1 : E;
+  const size_t per_row = ((size_t)n_logits + (scored ? E + sq.groups : 0)) * sizeof(float);
   const bool vec = D % 4 == 0 && (uintptr_t)router % 16 == 0;
-#define MOE_ROUTE_LAUNCH(TT, V)                                                                 \
-  if (scored) MOE_ROUTE_LAUNCH_AS(TT, V, true); else MOE_ROUTE_LAUNCH_AS(TT, V, false)
-#define MOE_ROUTE_LAUNCH_AS(TT, V, SQ)                                                          \
-  hipLaunchKernelGGL((moe_route_kernel<TT, V, SQ>), dim3(T), dim3(MOE_THREADS), lds, stream,      \
-                     (const TT*)x, ldx, router, bias, T, D, E, top, sq, gates, idx, wts)
+  // (rows that share a block must fit into its LDS together)
+  const bool wide = T <= MOE_ROUTE_WIDE_ROWS || MOE_ROUTE_SHARED_ROWS * per_row > 48 * 1024;
+  const int rows = wide ? 1 : MOE_ROUTE_SHARED_ROWS, threads = wide ? MOE_ROUTE_WIDE : MOE_THREADS;
+  // as many teams as there are groups of experts (up to four, a wave at least)
+  int teams = 1;
+  const int groups = (n_logits + MOE_ROUTE_GROUP - 1) / MOE_ROUTE_GROUP;
+  while (wide && teams < 4 && teams < groups) teams *= 2;
+  const size_t lds = rows * per_row +
+                     (size_t)rows * MOE_ROUTE_GROUP * (threads / WAVE) * sizeof(float);
+#define MOE_ROUTE_LAUNCH(TT, V)                                                                  \
+  if (scored) { MOE_ROUTE_LAUNCH_AS(TT, V, true) } else { MOE_ROUTE_LAUNCH_AS(TT, V, false) }
+#define MOE_ROUTE_LAUNCH_AS(TT, V, SC)                                                           \
+  if (wide) { MOE_ROUTE_LAUNCH_SHAPE(TT, V, SC, MOE_ROUTE_WIDE, 1); }                            \
+  else { MOE_ROUTE_LAUNCH_SHAPE(TT, V, SC, MOE_THREADS, MOE_ROUTE_SHARED_ROWS); }
+#define MOE_ROUTE_LAUNCH_SHAPE(TT, V, SC, TH, RO)                                                \
+  hipLaunchKernelGGL((moe_route_kernel<TT, V, SC, TH, RO>), dim3((T + RO - 1) / RO), dim3(TH),   \
+                     lds, stream, (const TT*)x, ldx, router, bias, T, D, E, top, teams, sq,      \
+                     gates, idx, wts)
   if (x_is_bf16) {
-    if (vec) { MOE_ROUTE_LAUNCH(bf16_t, 4); } else { MOE_ROUTE_LAUNCH(bf16_t, 1); }
+    if (vec) { MOE_ROUTE_LAUNCH(bf16_t, 4) } else { MOE_ROUTE_LAUNCH(bf16_t, 1) }
   } else {
-    if (vec) { MOE_ROUTE_LAUNCH(float, 4); } else { MOE_ROUTE_LAUNCH(float, 1); }
+    if (vec) { MOE_ROUTE_LAUNCH(float, 4) } else { MOE_ROUTE_LAUNCH(float, 1) }
   }
+#undef MOE_ROUTE_LAUNCH_SHAPE
 #undef MOE_ROUTE_LAUNCH_AS
 #undef MOE_ROUTE_LAUNCH
   KAPPAI_RETURN_LAUNCH_STATUS();

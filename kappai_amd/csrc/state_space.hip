@@ -334,9 +334,11 @@ __global__ __launch_bounds__(SS_THREADS) void state_space_carry_kernel(
   *reinterpret_cast<float4*>(st) = S;
 }
 
-// The chunks' outputs.  Grid as for the sums; a wave 16 rows of the chunk and the block's value
-// channels.
-#define SS_OUT_THREADS (SS_L / 16 * WAVE)
+// The chunks' outputs.  Grid as for the sums; a wave takes two tiles of 16 rows of the chunk, one near
+// its start and one near its end (a row meets as many of the chunk's rows as lie before it), and the
+// block's value channels.
+#define SS_TILES (SS_L / 16)
+#define SS_OUT_THREADS (SS_TILES / 2 * WAVE)
 template <int NS>
 __global__ __launch_bounds__(SS_OUT_THREADS) void state_space_out_kernel(
     const bf16_t* __restrict__ xbc, ss_columns at, const bf16_t* __restrict__ z, int z_stride,
@@ -354,17 +356,20 @@ __global__ __launch_bounds__(SS_OUT_THREADS) void state_space_out_kernel(
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
   const int row0 = chunks[3 * ch + 1], n = min(chunks[3 * ch + 2], SS_L), g = h / (H / G);
   const int lr = lane % 16, kg = lane / 16;
-  const int i0 = 16 * wave, i = i0 + lr;
+  const int first[2] = {16 * wave, 16 * (SS_TILES - 1 - wave)};
   // what only this wave reads is asked for first
-  ss_bf16x8_t cf[NS];
+  ss_bf16x8_t cf[2][NS];
 #pragma unroll
-  for (int s = 0; s < NS; ++s) {
-    uint4 q = make_uint4(0u, 0u, 0u, 0u);
-    if (i < n && 32 * s + 8 * kg < N)
-      q = *reinterpret_cast<const uint4*>(xbc + (size_t)(row0 + i) * at.stride + at.c_at + g * N +
-                                          32 * s + 8 * kg);
-    cf[s] = __builtin_bit_cast(ss_bf16x8_t, q);
-  }
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+      uint4 q = make_uint4(0u, 0u, 0u, 0u);
+      const int i = first[u] + lr;
+      if (i < n && 32 * s + 8 * kg < N)
+        q = *reinterpret_cast<const uint4*>(xbc + (size_t)(row0 + i) * at.stride + at.c_at +
+                                            g * N + 32 * s + 8 * kg);
+      cf[u][s] = __builtin_bit_cast(ss_bf16x8_t, q);
+    }
   ss_decays<false>(z, z_stride, row0, n, h, z_bias[h], rate[h], Ls, dts);
   ss_stage_turned(xbc, at.stride, at.x_at + h * dv + v0, row0, n, dv - v0, SS_V, Xt);
   for (int p = threadIdx.x; p < SS_L * 4 * NS; p += SS_OUT_THREADS) {
@@ -374,17 +379,14 @@ __global__ __launch_bounds__(SS_OUT_THREADS) void state_space_out_kernel(
       q = *reinterpret_cast<const uint4*>(xbc + (size_t)(row0 + j) * at.stride + at.b_at + g * N + e);
     *reinterpret_cast<uint4*>(Bs + j * BS + e) = q;
   }
-  __syncthreads();
-  if (i0 >= n) return;
-  const float Li = Ls[i];
-  ss_f32x4_t acc[VT];
-  // the state the chunk starts from, times the decay up to this row
+  // the state the chunk starts from (before the barrier: it needs nothing that is staged)
+  ss_f32x4_t acc[2][VT];
   const float* S0 = carry + (((size_t)ch * H + h) * dv + v0) * N;
 #pragma unroll
   for (int vt = 0; vt < VT; ++vt) {
-    acc[vt] = ss_f32x4_t{0.f, 0.f, 0.f, 0.f};
+    acc[0][vt] = acc[1][vt] = ss_f32x4_t{0.f, 0.f, 0.f, 0.f};
     const int v = 16 * vt + lr;
-    if (v0 + 16 * vt >= dv) continue;
+    if (v0 + 16 * vt >= dv || first[0] >= n) continue;
 #pragma unroll
     for (int s = 0; s < NS; ++s) {
       float w[8];
@@ -394,57 +396,67 @@ __global__ __launch_bounds__(SS_OUT_THREADS) void state_space_out_kernel(
       ss_bf16x8_t sf[3];
       ss_split(w, sf);
 #pragma unroll
-      for (int t = 0; t < 3; ++t) acc[vt] = ss_mfma(sf[t], cf[s], acc[vt]);
+      for (int t = 0; t < 3; ++t) {
+        acc[0][vt] = ss_mfma(sf[t], cf[0][s], acc[0][vt]);
+        acc[1][vt] = ss_mfma(sf[t], cf[1][s], acc[1][vt]);
+      }
     }
   }
-  const float fade = expf(Li);
+  __syncthreads();
 #pragma unroll
-  for (int vt = 0; vt < VT; ++vt)
+  for (int u = 0; u < 2; ++u) {
+    const int i0 = first[u], i = i0 + lr;
+    if (i0 >= n) continue;
+    // times the decay up to this row
+    const float Li = Ls[i], fade = expf(Li);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) acc[vt][r] *= fade;
-  // the chunk's own rows, 32 at a time
-  for (int jp = 0; jp <= i0; jp += 32) {
-    float p[8];
+    for (int vt = 0; vt < VT; ++vt)
 #pragma unroll
-    for (int jt = 0; jt < 2; ++jt) {
-      ss_f32x4_t gt = ss_f32x4_t{0.f, 0.f, 0.f, 0.f};
-      const bf16_t* bp = Bs + (jp + 16 * jt + lr) * BS + 8 * kg;
+      for (int r = 0; r < 4; ++r) acc[u][vt][r] *= fade;
+    // the chunk's own rows, 32 at a time
+    for (int jp = 0; jp <= i0; jp += 32) {
+      float p[8];
 #pragma unroll
-      for (int s = 0; s < NS; ++s)
-        gt = ss_mfma(__builtin_bit_cast(ss_bf16x8_t, *reinterpret_cast<const uint4*>(bp + 32 * s)),
-                     cf[s], gt);
-      const int j = jp + 16 * jt + 4 * kg;
-      const float4 l4 = *reinterpret_cast<const float4*>(Ls + j);
-      const float4 d4 = *reinterpret_cast<const float4*>(dts + j);
-      const float l[4] = {l4.x, l4.y, l4.z, l4.w}, d[4] = {d4.x, d4.y, d4.z, d4.w};
+      for (int jt = 0; jt < 2; ++jt) {
+        ss_f32x4_t gt = ss_f32x4_t{0.f, 0.f, 0.f, 0.f};
+        const bf16_t* bp = Bs + (jp + 16 * jt + lr) * BS + 8 * kg;
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        p[4 * jt + r] = j + r <= i ? gt[r] * (expf(Li - l[r]) * d[r]) : 0.f;
+        for (int s = 0; s < NS; ++s)
+          gt = ss_mfma(__builtin_bit_cast(ss_bf16x8_t, *reinterpret_cast<const uint4*>(bp + 32 * s)),
+                       cf[u][s], gt);
+        const int j = jp + 16 * jt + 4 * kg;
+        const float4 l4 = *reinterpret_cast<const float4*>(Ls + j);
+        const float4 d4 = *reinterpret_cast<const float4*>(dts + j);
+        const float l[4] = {l4.x, l4.y, l4.z, l4.w}, d[4] = {d4.x, d4.y, d4.z, d4.w};
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          p[4 * jt + r] = j + r <= i ? gt[r] * (expf(Li - l[r]) * d[r]) : 0.f;
+      }
+      ss_bf16x8_t pf[3];
+      ss_split(p, pf);
+#pragma unroll
+      for (int vt = 0; vt < VT; ++vt) {
+        const bf16_t* xp = Xt + (16 * vt + lr) * SS_LS + jp + 4 * kg;
+        const ss_bf16x8_t xf = ss_pieces(xp, xp + 16);
+#pragma unroll
+        for (int t = 0; t < 3; ++t) acc[u][vt] = ss_mfma(xf, pf[t], acc[u][vt]);
+      }
     }
-    ss_bf16x8_t pf[3];
-    ss_split(p, pf);
+    if (i >= n) continue;
+    const float sk = skip[h];
+    const bf16_t* xr = xbc + (size_t)(row0 + i) * at.stride + at.x_at + h * dv;
+    float* dst = out + ((size_t)(row0 + i) * H + h) * dv;
 #pragma unroll
     for (int vt = 0; vt < VT; ++vt) {
-      const bf16_t* xp = Xt + (16 * vt + lr) * SS_LS + jp + 4 * kg;
-      const ss_bf16x8_t xf = ss_pieces(xp, xp + 16);
-#pragma unroll
-      for (int t = 0; t < 3; ++t) acc[vt] = ss_mfma(xf, pf[t], acc[vt]);
+      const int v = v0 + 16 * vt + 4 * kg;
+      if (v >= dv) continue;
+      const uint2 q = *reinterpret_cast<const uint2*>(xr + v);
+      *reinterpret_cast<float4*>(dst + v) =
+          make_float4(fmaf(sk, __uint_as_float(q.x << 16), acc[u][vt][0]),
+                      fmaf(sk, __uint_as_float(q.x & 0xffff0000u), acc[u][vt][1]),
+                      fmaf(sk, __uint_as_float(q.y << 16), acc[u][vt][2]),
+                      fmaf(sk, __uint_as_float(q.y & 0xffff0000u), acc[u][vt][3]));
     }
-  }
-  if (i >= n) return;
-  const float sk = skip[h];
-  const bf16_t* xr = xbc + (size_t)(row0 + i) * at.stride + at.x_at + h * dv;
-  float* dst = out + ((size_t)(row0 + i) * H + h) * dv;
-#pragma unroll
-  for (int vt = 0; vt < VT; ++vt) {
-    const int v = v0 + 16 * vt + 4 * kg;
-    if (v >= dv) continue;
-    const uint2 q = *reinterpret_cast<const uint2*>(xr + v);
-    *reinterpret_cast<float4*>(dst + v) =
-        make_float4(fmaf(sk, __uint_as_float(q.x << 16), acc[vt][0]),
-                    fmaf(sk, __uint_as_float(q.x & 0xffff0000u), acc[vt][1]),
-                    fmaf(sk, __uint_as_float(q.y << 16), acc[vt][2]),
-                    fmaf(sk, __uint_as_float(q.y & 0xffff0000u), acc[vt][3]));
   }
 }
 

@@ -591,12 +591,15 @@ def _out_in_fragment_order(wanted: bool, M: int, N: int, force_kernel: int) -> b
 
 def linear_swiglu(x: torch.Tensor, weight: torch.Tensor, force_kernel: int = 0,
                   weight_frag: Optional[torch.Tensor] = None, out_fragment: bool = False,
-                  activation: int = 0):
+                  activation: int = 0, clamp: Optional["ClampedGate"] = None):
     """``silu(x Wg^T) * (x Wu^T)`` in one kernel: ``weight`` [2F, K] holds the gate and up
     matrices interleaved by ``interleave_gate_up``; bfloat16 only.  Returns [M, F].  ``x`` may
     be ``ScaledRows`` or ``FragmentRows``.  ``out_fragment``: with 8 to 16 rows the result may
     come back as ``FragmentRows`` for the product that follows.  ``activation``: ``GLU_SILU`` (0)
-    or ``GLU_GELU_TANH`` (1) in place of silu; the product kernels are built once per gate."""
+    or ``GLU_GELU_TANH`` (1) in place of silu, or ``GLU_CLAMPED`` (2) with its constants ``clamp``;
+    the product kernels are built once per gate."""
+    _need((activation == GLU_CLAMPED) == (clamp is not None),
+          "linear_swiglu: the clamped gate and its constants")
     scale = None
     if isinstance(x, ScaledRows):
         if (force_kernel not in (0, 2) or weight.dtype != BF16 or weight.dim() != 2
@@ -629,12 +632,12 @@ def linear_swiglu(x: torch.Tensor, weight: torch.Tensor, force_kernel: int = 0,
     c_frag = _out_in_fragment_order(out_fragment, M, F, force_kernel)
     out = torch.empty((16 if c_frag else M, F), dtype=BF16, device=x.device)
     gemm = library("gemm") if not activation else library("gemm", GATE_ACT=int(activation))
-    check(gemm.kappai_gemm_bf16_swiglu(
+    check(gemm.kappai_gemm_bf16_gated(
         _ptr(x), *_matrix(weight, weight_frag), _ptr(out), _c_int(M), _c_int(F), _c_int(K),
         _c_int(lda), _c_int(F),
         _c_int(force_kernel), _c_int(a_frag),
         *(scale._scale_args() if scale is not None else _NO_SCALE), _c_int(1 if c_frag else 0),
-        _stream()), "gemm_bf16_swiglu")
+        _ptr(clamp.on(x.device) if clamp else None), _stream()), "gemm_bf16_gated")
     return FragmentRows(out, M, None) if c_frag else out
 
 
@@ -1394,7 +1397,16 @@ class ClampedGate:
     def c_args(self):
         return _c_float(self.limit), _c_float(self.slope), _c_float(self.shift)
 
+    def on(self, device) -> torch.Tensor:
+        """The three constants as a float32 tensor there (made once)."""
+        key = (self, device)
+        if key not in _CLAMPS:
+            _CLAMPS[key] = torch.tensor([self.limit, self.slope, self.shift], dtype=F32,
+                                        device=device)
+        return _CLAMPS[key]
 
+
+_CLAMPS = {}
 _NO_CLAMP = (_c_float(0.0), _c_float(0.0), _c_float(0.0))
 
 

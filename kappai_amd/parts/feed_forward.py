@@ -36,8 +36,8 @@ class SwiGLU(FeedForward):
         """``activation``: what the gate passes through, "silu" or "gelu_tanh" (the tanh form of
         GELU): ``W_down (act(W_gate x + b_gate) * (W_up x + b_up)) + b_down``; or "clamped", the
         clamped gate with the constants ``clamp`` (``ops.ClampedGate``).  ``bias``: whether the three
-        maps have biases.  With biases or the clamped gate the gate runs as a kernel of its own
-        behind the first product."""
+        maps have biases (the gate then runs as a kernel of its own behind the first product, which
+        adds the biases)."""
         n = {"gate": "w1", "up": "w3", "down": "w2"}
         n.update(names or {})
         if activation not in self.ACTIVATIONS:
@@ -62,17 +62,20 @@ class SwiGLU(FeedForward):
         def interleaved(w):
             # the fused product wants gate and up rows in turns of 16
             self.fused = (w.dtype == torch.bfloat16 and self.hidden % ops.SWIGLU_GROUP == 0
-                          and self.width % 8 == 0 and not self.has_bias and self.clamp is None)
+                          and self.width % 8 == 0 and not self.has_bias)
             return ops.interleave_gate_up(w[:self.hidden], w[self.hidden:]) if self.fused else None
 
         self.gate_up.bind(tensors, arrange=interleaved)
+        if self.clamp is not None and self.gate_up.weight.device.type == "cuda":
+            self.clamp.on(self.gate_up.weight.device)      # (before any step is captured)
         self.down.bind(tensors)
 
     def forward(self, x, batch, into=None):
         if self.fused and x.dtype == torch.bfloat16:
             with profile.scope("matmul_ffn_gate_up", self.gate_up.weight_bytes()):
                 act = ops.linear_swiglu(x, self.gate_up.weight, out_fragment=True,
-                                        activation=self.ACTIVATIONS[self.activation])
+                                        activation=self.ACTIVATIONS[self.activation],
+                                        clamp=self.clamp)
             return self.down.forward(act, partial_sums=True, add_into=into)
         gate_up = self.gate_up.forward(x)
         with profile.scope("ffn_act"):

@@ -73,10 +73,13 @@ def interleave_gate_up(gate, up):
     return torch.cat([g, u], dim=1).reshape(2 * F, K).contiguous()
 
 
-def linear_swiglu(x, weight, force_kernel=0, weight_frag=None, out_fragment=False, activation=0):
+def linear_swiglu(x, weight, force_kernel=0, weight_frag=None, out_fragment=False, activation=0,
+                  clamp=None):
     F = weight.shape[0] // 2
     y = (x.to(F32) @ weight.to(F32).T).reshape(x.shape[0], F // SWIGLU_GROUP, 2, SWIGLU_GROUP)
     g, u = y[:, :, 0, :].reshape(-1, F), y[:, :, 1, :].reshape(-1, F)
+    if activation == 2:
+        return _clamped(g, u, clamp).to(x.dtype)
     if activation == 1:
         a = 0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g ** 3)))
     else:

@@ -407,6 +407,28 @@ def test_clamped_gate_of_a_dense_product(dtype, tol, F):
         ops.glu(x.to(DEV), ops.GLU_CLAMPED)
 
 
+@pytest.mark.parametrize("M", [1, 8, 16, 20, 33, 64, 100, 300, 2100])
+@pytest.mark.parametrize("F,K", [(64, 64), (48, 72), (512, 256)])
+def test_clamped_gate_in_the_epilogue_of_a_product(M, F, K):
+    """Every form of the gated product kernels, at row counts that select each, against its formula;
+    inputs wide enough for the limit to bite on both sides."""
+    from kappai_amd.kernels import ops
+    g = gen(M + F)
+    x = torch.randn(M, K, generator=g).to(BF16)
+    wg, wu = ((torch.randn(F, K, generator=g) * 2 / math.sqrt(K)).to(BF16) for _ in range(2))
+    w = ops.interleave_gate_up(wg, wu).to(DEV)
+    a, b = x.double() @ wg.double().T, x.double() @ wu.double().T
+    a, b = a.clamp(max=1.3), b.clamp(-1.3, 1.3)
+    want = a * torch.sigmoid(1.6 * a) * (b + 0.75)
+    clamp = ops.ClampedGate(1.3, 1.6, 0.75)
+    forms = [w] + ([ops.InFragments.of(w)] if ops.InFragments.of(w) is not None else [])
+    for m in forms:
+        got = ops.linear_swiglu(x.to(DEV), m, activation=ops.GLU_CLAMPED, clamp=clamp)
+        assert rel(got.float(), want) < 1e-2
+    with pytest.raises(ValueError, match="constants"):
+        ops.linear_swiglu(x.to(DEV), w, activation=ops.GLU_CLAMPED)
+
+
 # ---------------------------------------------------------------------------------------------
 # parts
 # ---------------------------------------------------------------------------------------------
