@@ -471,7 +471,7 @@ __global__ __launch_bounds__(8 * WAVE) void attn_prefill_shared_kernel(
     const bf16_t* __restrict__ vt_pool, bf16_t* __restrict__ out, int out_stride,
     const int* __restrict__ q_tiles, const int* __restrict__ row_pos,
     const int* __restrict__ block_tables, int max_blocks, int H, int G, int ps, int window,
-    float scale) {
+    float scale, const float* __restrict__ sink) {
   constexpr int ROWB = HEAD_DIM * 2;                // bytes of a key's row
   constexpr int KTILE = 32 * ROWB, VGROUP = HEAD_DIM * 32, BUF = KTILE + 2 * VGROUP;   // bytes
   constexpr int CPR = ROWB / 16;                    // 16-byte chunks a K row
@@ -840,7 +840,8 @@ __global__ __launch_bounds__(8 * WAVE) void attn_prefill_shared_kernel(
     if (it + 2 < n_steps) step(PgBuf<2>{}, it + 2);
   }
   if (!row_ok) return;
-  const float l_run = MFMA_SUM ? o_sum[0] : l_add;
+  float l_run = MFMA_SUM ? o_sum[0] : l_add;
+  if (sink != nullptr && m_ref != -INFINITY) l_run += fast_exp2(sink[h] * LOG2E - m_ref);
   const float inv = l_run > 0.f ? 1.0f / l_run : 0.f;
   bf16_t* orow = out + (size_t)(r0 + col) * out_stride + (size_t)h * HEAD_DIM;
 #pragma unroll
@@ -1581,18 +1582,16 @@ extern "C" int kappai_attn_prefill_scored(const void* q, int q_stride, const voi
     return (int)hipErrorInvalidValue;
   const int rep = H / G;
   const bool shared_ok = PG_OK && rep % 4 == 0;
-  if (variant == 2 && (!shared_ok || sink != nullptr)) return (int)hipErrorInvalidValue;
+  if (variant == 2 && !shared_ok) return (int)hipErrorInvalidValue;
   // sharing pays when there are blocks enough to fill the chip without splitting the keys of
   // a q tile over waves
-  // (the kernel that shares key tiles knows no sink)
-  const bool shared = variant == 2 ||
-                      (variant == 0 && shared_ok && sink == nullptr && n_tiles * (H / 4) >= 256);
+  const bool shared = variant == 2 || (variant == 0 && shared_ok && n_tiles * (H / 4) >= 256);
 #if PG_OK
   if (shared) {
     hipLaunchKernelGGL(attn_prefill_shared_kernel, dim3(n_tiles, H / 4), dim3(8 * WAVE), 0, stream,
                        (const bf16_t*)q, q_stride, (const bf16_t*)k_pool, (const bf16_t*)vt_pool,
                        (bf16_t*)out, out_stride, q_tiles, row_pos, block_tables, max_blocks, H, G,
-                       ps, window, scale);
+                       ps, window, scale, sink);
     KAPPAI_RETURN_LAUNCH_STATUS();
   }
 #endif

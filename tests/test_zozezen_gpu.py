@@ -473,6 +473,42 @@ def test_attention_with_keys_of_its_own_and_on_another_layers(dtype, tol, H, G, 
     assert float((want - want2).abs().max()) > 0.2 * float(want.abs().max())
 
 
+@pytest.mark.parametrize("variant", [1, 2])
+@pytest.mark.parametrize("H,G,d", [(8, 2, 64), (4, 1, 64), (8, 1, 128), (16, 4, 128)])
+def test_a_sink_in_both_forms_of_the_prompt_kernel(variant, H, G, d):
+    """The tiled kernel whose blocks share key tiles among four heads, and the one of a block a head,
+    with a sink a head from negligible to overwhelming; portions that start at a page's border and
+    in the middle of one."""
+    from kappai_amd.kernels import ops
+    N, ps, scale = 300, 16, 1.0 / math.sqrt(d)
+    g = gen(H + d)
+    q, k, v = (torch.randn(N, n, d, generator=g).to(BF16) for n in (H, G, G))
+    sink = torch.linspace(-60.0, 9.0, H)
+    sink[1] = 0.0
+    n_pages = (N + ps - 1) // ps
+    order = torch.randperm(n_pages, generator=g)
+    kp = torch.full((n_pages, G, ps, d), float("nan"), dtype=BF16)
+    vp = torch.full((n_pages, G, d, ps), float("nan"), dtype=BF16)
+    for p in range(N):
+        kp[order[p // ps], :, p % ps] = k[p]
+        vp[order[p // ps], :, :, p % ps] = v[p]
+    kk, vv = (x.double().repeat_interleave(H // G, dim=1) for x in (k, v))
+    sc = torch.einsum("ihd,jhd->hij", q.double(), kk) * scale
+    sc = sc.masked_fill(torch.arange(N)[None, :] > torch.arange(N)[:, None], -math.inf)
+    w = torch.softmax(torch.cat([sc, sink.double()[:, None, None].expand(-1, N, 1)], 2), 2)[..., :-1]
+    want = torch.einsum("hij,jhd->ihd", w, vv).reshape(N, -1)
+    for start, n in ((0, N), (32, 200), (77, 33), (N - 2, 2)):
+        nt = (n + 31) // 32
+        tiles = [[0, 32 * i, min(32, n - 32 * i), i | (nt << 16)] for i in range(nt)]
+        i32 = lambda x: torch.tensor(x, dtype=I32, device=DEV)
+        got = ops.paged_attention(
+            q[start:start + n].reshape(n, H * d).to(DEV), H, G, d, kp.to(DEV), vp.to(DEV),
+            i32(list(range(start, start + n))), i32([0] * n), order.to(I32)[None].to(DEV), ps, scale,
+            q_tiles=i32(tiles), max_position=start + n - 1, kernel="prefill",
+            prefill_variant=variant, mods=ops.ScoreMods(0.0, None, sink.to(DEV)))
+        assert rel(got.float(), want[start:start + n]) < 2e-2, (start, n)
+
+
 def needle_case(H, d, dtype, scale):
     """A part whose queries read the first half of the input and whose keys and values read the second,
     one for one; norm weights of one and open gates."""
